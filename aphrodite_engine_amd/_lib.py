@@ -168,18 +168,21 @@ MIXERS_LIB_PATH = os.environ.get(
     "APHRODITE_MI355X_MIXERS_LIB", os.path.join(_HERE, "lib", "libaphrodite_mi355x_mixers.so"))
 MIXERS_SIGNATURES = {
     "aphro_mixers_last_error": (ctypes.c_char_p, []),
-    "aphro_embed_scale_f32": (I, [P, P, P, L, I, L, F, I, P]),
+    "aphro_embed_scale_f32": (I, [P, P, P, L, I, L, F, P, I, P]),
     "aphro_residual_layer_norm": (I, [P, P, L, P, P, P, P, P, P, P, L, I, F, I, P]),
     "aphro_act_and_mul": (I, [P, P, L, L, I, I, I, P]),
     "aphro_gated_group_rms_norm": (I, [P, L, P, P, P, L, L, I, I, F, F, I, P]),
     "aphro_paged_kv_write": (I, [P, P, P, L, P, L, P, L, I, I, I, L, I, P]),
     "aphro_distance_bias_attention": (I, [P, L, P, L, P, L, P, P, P, I, L, I, P, P, P, P, L, I, I, I, I, I, I, I, F, P, I, F,
-                                          I, F, I, P, L, I, P]),
-    "aphro_outer_memory_scan": (I, [P, P, L, P, L, P, L, P, P, L, P, P, P, P, I, P, P, P, I, L, I, I, I, I, P, F, F, I, I, P]),
+                                          I, F, I, I, F, P, I, I, P, L, I, P]),
+    "aphro_residual_post_rms_norm": (I, [P, P, L, P, P, P, L, I, F, I, P]),
+    "aphro_silu_gate_part_rms_norm": (I, [P, L, P, P, L, P, L, I, I, F, F, I, P]),
+    "aphro_qk_row_norm_kv_write": (I, [P, L, P, P, P, L, P, L, P, L, P, L, P, P, L, I, I, I, F, I, P]),
+    "aphro_outer_memory_scan": (I, [P, P, L, P, L, P, L, P, P, L, P, P, P, P, I, P, P, P, I, L, I, I, I, I, P, F, F, I, P, P, P, I, I, P]),
     "aphro_depth_residual_rms_norm": (I, [P, P, P, L, P, L, I, P, F, P, P, L, I, F, I, P]),
     "aphro_poly_norm": (I, [P, P, L, L, I, F, F, F, F, F, I, P]),
     "aphro_differential_norm_gate": (I, [P, L, P, L, P, L, L, I, I, I, F, F, F, I, P]),
-    "aphro_short_conv": (I, [P, L, P, P, P, L, P, L, P, P, P, P, P, P, P, L, I, I, I, I, I, I, I, P]),
+    "aphro_short_conv": (I, [P, L, P, P, P, L, P, L, P, P, P, P, P, P, P, P, L, I, I, I, I, I, I, I, P]),
     "aphro_windowed_attention": (I, [P, L, P, L, P, P, P, I, L, I, P, P, P, P, L, I, I, I, I, I, I, I, I, F, I, I, I, P, L, I, P]),
     "aphro_differential_window_attention_supported": (I, [I, I, I, I, I]),
     "aphro_differential_window_attention": (I, [P, L, P, L, P, L, P, P, P, I, L, I, P, P, P, P, L, I, I, I, I, I, I, I, F, I, I, F, F,
@@ -205,9 +208,9 @@ MIXERS_SIGNATURES = {
     "aphro_experts_route_topk": (I, [P, P, P, P, L, I, I, P]),
     "aphro_hyper_residual_rms_norm": (I, [P, P, L, P, P, P, F, P, P, P, P, L, I, I, F, I, P]),
     "aphro_logit_softcap": (I, [P, P, L, F, F, I, P]),
-    "aphro_gated_delta_scan": (I, [P, P, L, P, L, P, L, P, L, P, L, P, P, P, P, I, P, P, P, I, L, I, I, I, I, F, F, I, I, P]),
+    "aphro_gated_delta_scan": (I, [P, P, L, P, L, P, L, P, L, P, L, P, P, P, P, I, P, P, P, I, L, I, I, I, I, I, F, F, I, I, P]),
     "aphro_gated_head_rms_norm": (I, [P, L, P, P, P, L, L, I, I, F, I, I, P]),
-    "aphro_rotary_qk_norm_kv_write": (I, [P, L, P, P, P, L, P, L, P, L, P, L, P, L, F, P, P, P, P, L, I, I, I, I, I, I, I, F, I, P]),
+    "aphro_rotary_qk_norm_kv_write": (I, [P, L, P, P, P, L, P, L, P, L, P, L, P, L, F, P, P, P, P, L, I, I, I, I, I, I, I, P, P, F, I, P]),
 }
 
 OK = 0

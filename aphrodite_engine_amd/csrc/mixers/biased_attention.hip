@@ -1,12 +1,14 @@
 // Softmax attention over a token-major paged cache with a tabulated distance bias, a position-dependent query
 // temperature and a per-head sigmoid output gate -- one kernel for prompt portions and single decoded tokens (a batch
-// is a list of segments; every query row attends to keys 0 .. its own position, all read from the cache).
+// is a list of segments; every query row attends to keys 0 .. its own position, all read from the cache).  Optional: a
+// sliding window, chunks counted from the sequence's start (a row sees its own chunk only), a tanh soft cap on the scores
+// before the bias, a per-head sink (a score without key or value) in the softmax denominator, an elementwise gate.
 //
 // Work split: one workgroup of four waves per (query row, head).  The waves take the 64-key tiles round-robin; inside a
 // tile lane = key for the scores (fp32 dot product, online softmax with wave-wide max / sum), then lane = output column
 // for P V (the probability of key jj is broadcast with v_readlane).  The four partial (max, sum, accumulator) triples
 // are merged through LDS.  Scores, softmax and the accumulators are fp32 whatever the storage type.
-#include "mixers_common.h"
+#include "biased_attention.h"
 
 namespace aphro {
 
@@ -63,13 +65,17 @@ __global__ __launch_bounds__(256) void distance_bias_attention_kernel(
     const typename T::storage* __restrict__ v_cache, const int32_t* __restrict__ block_tables, int max_blocks,
     int64_t num_blocks, int block_size, const int32_t* __restrict__ q_start, const int32_t* __restrict__ ctx_len,
     const int32_t* __restrict__ seq_of_token, int heads, int kv_heads, int dim, int vdim, float scale,
-    const float* __restrict__ bias_lut, int lut_len, float temp_coef, int temp_every, float out_scale) {
+    const float* __restrict__ bias_lut, int lut_len, float temp_coef, int temp_every, float out_scale, int window, int chunk,
+    float softcap, const float* __restrict__ sink, int gate_cols) {
   __shared__ __attribute__((aligned(16))) float qsh[DBA_MAX_DIM];
   __shared__ float merge[DBA_WAVES][2 + EPL * 64];
   const int t = blockIdx.x, h = blockIdx.y;
   const int s = seq_of_token[t];
   const int pos = ctx_len[s] + (t - q_start[s]);
   const int nkeys = pos + 1;
+  int lo = 0;                                               // oldest visible key
+  if (window > 0) lo = max(lo, pos - window + 1);
+  if (chunk > 0) lo = max(lo, pos / chunk * chunk);
   const int g = h / (heads / kv_heads);
   const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
   float qs = scale;
@@ -83,14 +89,15 @@ __global__ __launch_bounds__(256) void distance_bias_attention_kernel(
 #pragma unroll
   for (int c = 0; c < EPL; ++c) acc[c] = 0.f;
   const int ntiles = (nkeys + 63) >> 6;
-  for (int tile = wave; tile < ntiles; tile += DBA_WAVES) {
+  for (int tile = (lo >> 6) + wave; tile < ntiles; tile += DBA_WAVES) {
     const int j = tile * 64 + lane;
     float sc = -INFINITY;
-    if (j < nkeys) {
+    if (j >= lo && j < nkeys) {
       const int blk = bt[j / block_size];
       if (blk >= 0 && blk < num_blocks) {
         const typename T::storage* kr = k_cache + ((int64_t)blk * block_size + j % block_size) * krow + g * dim;
         sc = dot_row<T>(qsh, kr, dim) * qs;
+        if (softcap > 0.f) sc = softcap * tanhf(sc / softcap);
         if (lut) {
           const int dist = pos - j;
           sc += lut[dist < lut_len ? dist : lut_len - 1];
@@ -106,7 +113,7 @@ __global__ __launch_bounds__(256) void distance_bias_attention_kernel(
     for (int c = 0; c < EPL; ++c) acc[c] *= alpha;
     const int cnt = min(64, nkeys - tile * 64);
 #pragma unroll 4
-    for (int jj = 0; jj < cnt; ++jj) {
+    for (int jj = max(0, lo - tile * 64); jj < cnt; ++jj) {
       const float pj = __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, p), jj));
       const int j2 = tile * 64 + jj;
       int blk = bt[j2 / block_size];
@@ -130,14 +137,15 @@ __global__ __launch_bounds__(256) void distance_bias_attention_kernel(
   float M = -INFINITY;
 #pragma unroll
   for (int w = 0; w < DBA_WAVES; ++w) M = fmaxf(M, merge[w][0]);
-  float L = 0.f, f[DBA_WAVES];
+  if (sink) M = fmaxf(M, sink[h]);
+  float L = sink ? expf(sink[h] - M) : 0.f, f[DBA_WAVES];
 #pragma unroll
   for (int w = 0; w < DBA_WAVES; ++w) {
     f[w] = (merge[w][0] == -INFINITY) ? 0.f : expf(merge[w][0] - M);
     L += merge[w][1] * f[w];
   }
   float sig = out_scale;
-  if (gate) sig *= sigmoid_f(T::to_f32(gate[(int64_t)t * gate_stride + h]));
+  if (gate && !gate_cols) sig *= sigmoid_f(T::to_f32(gate[(int64_t)t * gate_stride + h]));
   const float inv = sig / L;
 #pragma unroll
   for (int c = 0; c < EPL; ++c) {
@@ -146,37 +154,12 @@ __global__ __launch_bounds__(256) void distance_bias_attention_kernel(
       float o = 0.f;
 #pragma unroll
       for (int w = 0; w < DBA_WAVES; ++w) o += merge[w][2 + col] * f[w];
-      out[(int64_t)t * out_stride + h * vdim + col] = T::from_f32(o * inv);
+      o *= inv;
+      if (gate && gate_cols) o *= sigmoid_f(T::to_f32(gate[(int64_t)t * gate_stride + h * vdim + col]));
+      out[(int64_t)t * out_stride + h * vdim + col] = T::from_f32(o);
     }
   }
 }
-
-// biased_attention_fast.hip
-struct DBAParams {
-  uint16_t* out;
-  const uint16_t* q;
-  const uint16_t* gate;
-  const uint16_t* k_cache;
-  const uint16_t* v_cache;
-  const int32_t* block_tables;
-  const int32_t* q_start;
-  const int32_t* q_len;
-  const int32_t* ctx_len;
-  const int32_t* seq_of_token;
-  const float* bias_lut;
-  int64_t out_stride, q_stride, gate_stride, num_blocks;
-  int max_blocks, block_size, heads, kv_heads, dim, vdim, lut_len, temp_every, min_len;
-  float scale, temp_coef, out_scale;
-  float* ws;
-  int bs_shift;
-  int max_tiles;
-};
-bool dba_prefill_supported(int dim, int vdim);
-bool dba_decode_supported(int heads, int kv_heads, int dim, int vdim);
-void dba_prefill_launch(const DBAParams& p, int max_q_len, int num_seqs, hipStream_t st);
-void dba_decode_launch(const DBAParams& p, int64_t num_tokens, int nsplit, hipStream_t st);
-int dba_decode_splits(int64_t num_tokens, int kv_heads, int max_kv_len, int64_t ws_floats, int heads, int vdim);
-constexpr int DBA_MFMA_MIN_LEN = 8;     // segments at least this long go to the matrix-core kernel
 
 }  // namespace aphro
 
@@ -206,8 +189,8 @@ extern "C" int aphro_distance_bias_attention(void* out, int64_t out_stride, cons
                                              const int32_t* seq_of_token, int64_t num_tokens, int num_seqs, int min_q_len,
                                              int max_q_len, int heads, int kv_heads, int dim, int vdim, float scale,
                                              const float* bias_lut, int lut_len, float temp_coef, int temp_every,
-                                             float out_scale, int max_kv_len, float* workspace, int64_t workspace_floats,
-                                             int dtype, void* stream) {
+                                             float out_scale, int window, int chunk, float softcap, const float* sink, int gate_cols,
+                                             int max_kv_len, float* workspace, int64_t workspace_floats, int dtype, void* stream) {
   if (num_tokens == 0) return APHRO_OK;
   APHRO_CHECK(out && q && k_cache && v_cache && block_tables && q_start && ctx_len && seq_of_token,
               "distance_bias_attention: null argument");
@@ -216,10 +199,16 @@ extern "C" int aphro_distance_bias_attention(void* out, int64_t out_stride, cons
   APHRO_CHECK(dim > 0 && dim <= DBA_MAX_DIM && vdim > 0 && vdim <= DBA_MAX_VDIM,
               "distance_bias_attention: dim %d (<= %d) / vdim %d (<= %d)", dim, DBA_MAX_DIM, vdim, DBA_MAX_VDIM);
   APHRO_CHECK(block_size > 0 && max_blocks > 0 && num_blocks > 0 && num_seqs > 0, "distance_bias_attention: bad cache geometry");
-  APHRO_CHECK(q_stride >= (int64_t)heads * dim && out_stride >= (int64_t)heads * vdim && (!gate || gate_stride >= heads),
+  APHRO_CHECK(q_stride >= (int64_t)heads * dim && out_stride >= (int64_t)heads * vdim && (!gate || gate_stride >= (gate_cols ? (int64_t)heads * vdim : (int64_t)heads)),
               "distance_bias_attention: row strides smaller than the rows");
   APHRO_CHECK(!bias_lut || lut_len > 0, "distance_bias_attention: empty bias table");
   APHRO_CHECK(temp_coef == 0.f || temp_every > 0, "distance_bias_attention: temp_every must be positive");
+  APHRO_CHECK(window >= 0 && chunk >= 0 && softcap >= 0.f && (gate_cols == 0 || gate_cols == 1), "distance_bias_attention: window %d, chunk %d, cap %g",
+              window, chunk, softcap);
+  const bool ext = window > 0 || chunk > 0 || softcap > 0.f || sink || (gate && gate_cols);
+  int visible = max_kv_len;                                 // what a row can see, not how long its sequence is, decides the split
+  if (window > 0) visible = min(visible, window);
+  if (chunk > 0) visible = min(visible, chunk);
   // bf16 with 16-byte-aligned rows: the matrix-core kernel for the long segments, the shared-key kernel for the rest
   if (dtype == APHRO_BF16 && q_len && max_q_len >= min_q_len && min_q_len > 0 && ((uintptr_t)q & 15) == 0 && (q_stride & 7) == 0) {
     DBAParams p;
@@ -231,23 +220,32 @@ extern "C" int aphro_distance_bias_attention(void* out, int64_t out_stride, cons
     p.lut_len = lut_len; p.temp_every = temp_every; p.scale = scale; p.temp_coef = temp_coef; p.out_scale = out_scale;
     p.ws = workspace;
     p.max_tiles = 0;
+    p.window = window; p.chunk = chunk; p.softcap = softcap; p.sink = sink; p.gate_cols = gate_cols;
+    p.cap_in = softcap > 0.f ? 2.0f / softcap : 0.f;
+    p.cap_out = softcap * 1.4426950408889634f;
+    p.vec4 = (out_stride & 3) == 0 && ((uintptr_t)out & 7) == 0 && (!gate || ((gate_stride & 3) == 0 && ((uintptr_t)gate & 7) == 0));
     p.bs_shift = -1;
     for (int sft = 0; sft < 20; ++sft)
       if ((1 << sft) == block_size) p.bs_shift = sft;
-    const int nsplit = workspace ? dba_decode_splits(num_tokens, kv_heads, max_kv_len, workspace_floats, heads, vdim) : 1;
+    const int nsplit = workspace ? dba_decode_splits(num_tokens, dba_decode_units(heads, kv_heads, dim, vdim), visible, workspace_floats, heads, vdim) : 1;
     const bool pf = dba_prefill_supported(dim, vdim) && max_q_len >= DBA_MFMA_MIN_LEN;
     const bool dc = dba_decode_supported(heads, kv_heads, dim, vdim);
     const bool all_long = min_q_len >= DBA_MFMA_MIN_LEN;
     if (pf && (all_long || dc)) {
       p.min_len = DBA_MFMA_MIN_LEN;
-      dba_prefill_launch(p, max_q_len, num_seqs, (hipStream_t)stream);
-      if (!all_long) dba_decode_launch(p, num_tokens, nsplit, (hipStream_t)stream);
+      if (ext) dba_prefill_launch<true>(p, max_q_len, num_seqs, (hipStream_t)stream);
+      else dba_prefill_launch<false>(p, max_q_len, num_seqs, (hipStream_t)stream);
+      if (!all_long) {
+        if (ext) dba_decode_launch<true>(p, num_tokens, nsplit, (hipStream_t)stream);
+        else dba_decode_launch<false>(p, num_tokens, nsplit, (hipStream_t)stream);
+      }
       APHRO_LAUNCH_CHECK();
       return APHRO_OK;
     }
     if (dc) {
       p.min_len = 0x7fffffff;
-      dba_decode_launch(p, num_tokens, nsplit, (hipStream_t)stream);
+      if (ext) dba_decode_launch<true>(p, num_tokens, nsplit, (hipStream_t)stream);
+      else dba_decode_launch<false>(p, num_tokens, nsplit, (hipStream_t)stream);
       APHRO_LAUNCH_CHECK();
       return APHRO_OK;
     }
@@ -258,7 +256,7 @@ extern "C" int aphro_distance_bias_attention(void* out, int64_t out_stride, cons
   hipLaunchKernelGGL((distance_bias_attention_kernel<T, EPL>), grid, dim3(256), 0, (hipStream_t)stream, (S*)out, out_stride, \
                      (const S*)q, q_stride, (const S*)gate, gate_stride, (const S*)k_cache, (const S*)v_cache, block_tables,  \
                      max_blocks, num_blocks, block_size, q_start, ctx_len, seq_of_token, heads, kv_heads, dim, vdim, scale,  \
-                     bias_lut, lut_len, temp_coef, temp_every, out_scale)
+                     bias_lut, lut_len, temp_coef, temp_every, out_scale, window, chunk, softcap, sink, gate_cols)
   MIX_DISPATCH_DTYPE(dtype, {
     typedef typename T::storage S;
     switch (epl) {

@@ -1,13 +1,15 @@
 // Gated delta rule: per (request slot, head) a matrix state S [dim, vdim] that forgets, corrects what it holds under the key
 // towards the new value, and is read AFTER the write:
 //     S <- g_t S;   u_t = beta_t (v_t - S^T k_t);   S <- S + k_t u_t^T;   o_t = S^T q_t
+// (CHANNEL form: g_t is a vector over the key dimension, one decay per row of S: g_t[r] = exp(-exp(A_log) softplus(a_t[r] + dt_bias[r])))
 // with k and q made unit vectors per head (x / sqrt(sum x^2 + norm_eps); q times q_scale), beta_t = sigmoid(b_t) and
 // g_t = exp(-exp(A_log) * softplus(a_t + dt_bias)) per head.  State, the unit norms, beta, g and every sum are fp32 whatever
 // the activations' storage.  Query / key head of value head h: h / (heads / kv_heads).
 //
 // With r_k = S_old^T k and r_q = S_old^T q (ONE pass over the state, two dot products per column):
 //     u = beta (v - g r_k),   S_new = g S_old + k u^T,   o = g r_q + (k . q) u
-// so a token costs one read pass and one update pass over the registers that hold the state.
+// so a token costs one read pass and one update pass over the registers that hold the state.  In the CHANNEL form the read pass
+// decays the rows as it goes (S <- g S, r_k = S^T k, r_q = S^T q) and the update adds k u^T: the same number of operations.
 //
 // Work split (that of the gated outer-product memories): a workgroup of 256 threads owns 64 -- for prompt portions 16 -- value
 // columns of one (segment, head); thread = (column, slice of the key dimension); 16 tokens at a time are staged in LDS, sixteen
@@ -21,9 +23,7 @@ namespace aphro {
 
 constexpr int GDR_CH = 16;
 
-__device__ __forceinline__ float softplus_f(float z) { return z > 20.f ? z : log1pf(expf(z)); }
-
-template <typename T, int DPT, int SLOG>
+template <typename T, int DPT, int SLOG, bool CHANNEL>
 __global__ __launch_bounds__(256) void gated_delta_scan_kernel(
     float* __restrict__ out, const typename T::storage* __restrict__ q, int64_t q_stride,
     const typename T::storage* __restrict__ k, int64_t k_stride, const typename T::storage* __restrict__ v, int64_t v_stride,
@@ -39,6 +39,7 @@ __global__ __launch_bounds__(256) void gated_delta_scan_kernel(
   constexpr int NV = (GDR_CH * TW + 255) / 256;
   __shared__ __attribute__((aligned(16))) float qs[GDR_CH][DP];
   __shared__ __attribute__((aligned(16))) float ks[GDR_CH][DP];
+  __shared__ __attribute__((aligned(16))) float gs[CHANNEL ? GDR_CH : 1][CHANNEL ? DP : 1];
   __shared__ float vs[GDR_CH][TW];
   __shared__ float g_s[GDR_CH], b_s[GDR_CH], kq_s[GDR_CH];
   const int s = blockIdx.x, h = blockIdx.y, c0 = blockIdx.z * TW;
@@ -56,10 +57,18 @@ __global__ __launch_bounds__(256) void gated_delta_scan_kernel(
     const int r = sl * DPT + i;
     S[i] = (!fresh && r < dim && col < vdim) ? sbase[(int64_t)r * vdim + col] : 0.f;
   }
-  const float neg_rate = -expf(a_log[h]), dtb = dt_bias[h];
+  const float neg_rate = -expf(a_log[h]), dtb = CHANNEL ? 0.f : dt_bias[h];
   const int stok = tid >> 4, sln = tid & 15;               // staging: token of the stage, lane within the token
 
   float rq[NQ], rk[NQ], rv[NV], rb = 0.f, ra = 0.f;
+  float rg[CHANNEL ? NQ : 1], dtc[CHANNEL ? NQ : 1];       // per-channel decay: raw values of the next stage, the lane's dt_bias
+  if constexpr (CHANNEL) {
+#pragma unroll
+    for (int it = 0; it < NQ; ++it) {
+      const int r = sln + 16 * it;
+      dtc[it] = r < dim ? dt_bias[h * dim + r] : 0.f;
+    }
+  }
   auto fetch = [&](int base) {
     const int cnt = min(GDR_CH, n - base);
 #pragma unroll
@@ -69,6 +78,9 @@ __global__ __launch_bounds__(256) void gated_delta_scan_kernel(
       if (stok < cnt && r < dim) {
         rq[it] = T::to_f32(q[(t0 + base + stok) * q_stride + hk * dim + r]);
         rk[it] = T::to_f32(k[(t0 + base + stok) * k_stride + hk * dim + r]);
+        if constexpr (CHANNEL) rg[it] = T::to_f32(a[(t0 + base + stok) * a_stride + (int64_t)h * dim + r]);
+      } else if constexpr (CHANNEL) {
+        rg[it] = 0.f;
       }
     }
 #pragma unroll
@@ -78,7 +90,7 @@ __global__ __launch_bounds__(256) void gated_delta_scan_kernel(
     }
     if (sln == 0 && stok < cnt) {
       rb = T::to_f32(b[(t0 + base + stok) * b_stride + h]);
-      ra = T::to_f32(a[(t0 + base + stok) * a_stride + h]);
+      if constexpr (!CHANNEL) ra = T::to_f32(a[(t0 + base + stok) * a_stride + h]);
     }
   };
   fetch(0);
@@ -104,13 +116,14 @@ __global__ __launch_bounds__(256) void gated_delta_scan_kernel(
         if (r < DP) {
           qs[stok][r] = qv;
           ks[stok][r] = kv;
+          if constexpr (CHANNEL) gs[stok][r] = expf(neg_rate * softplus_f(rg[it] + dtc[it]));
         }
       }
       kq = group_sum<4>(kq);
       if (sln == 0) {
         kq_s[stok] = kq;
         b_s[stok] = sigmoid_f(rb);
-        g_s[stok] = expf(neg_rate * softplus_f(ra + dtb));
+        if constexpr (!CHANNEL) g_s[stok] = expf(neg_rate * softplus_f(ra + dtb));
       }
     }
 #pragma unroll
@@ -122,12 +135,17 @@ __global__ __launch_bounds__(256) void gated_delta_scan_kernel(
     if (base + GDR_CH < n) fetch(base + GDR_CH);
 #pragma unroll 2
     for (int tt = 0; tt < cnt; ++tt) {
-      const float g = g_s[tt], beta = b_s[tt], kq = kq_s[tt];
+      const float g = CHANNEL ? 1.f : g_s[tt], beta = b_s[tt], kq = kq_s[tt];
       float pk[4] = {0.f, 0.f, 0.f, 0.f}, pq[4] = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
       for (int i4 = 0; i4 < DPT; i4 += 4) {
         const f32x4 kk = *reinterpret_cast<const f32x4*>(&ks[tt][sl * DPT + i4]);
         const f32x4 qq = *reinterpret_cast<const f32x4*>(&qs[tt][sl * DPT + i4]);
+        if constexpr (CHANNEL) {
+          const f32x4 gg = *reinterpret_cast<const f32x4*>(&gs[tt][sl * DPT + i4]);
+#pragma unroll
+          for (int e = 0; e < 4; ++e) S[i4 + e] *= gg[e];
+        }
 #pragma unroll
         for (int e = 0; e < 4; ++e) {
           pk[e] += S[i4 + e] * kk[e];
@@ -141,7 +159,7 @@ __global__ __launch_bounds__(256) void gated_delta_scan_kernel(
       for (int i4 = 0; i4 < DPT; i4 += 4) {
         const f32x4 kk = *reinterpret_cast<const f32x4*>(&ks[tt][sl * DPT + i4]);
 #pragma unroll
-        for (int e = 0; e < 4; ++e) S[i4 + e] = g * S[i4 + e] + kk[e] * u;
+        for (int e = 0; e < 4; ++e) S[i4 + e] = (CHANNEL ? S[i4 + e] : g * S[i4 + e]) + kk[e] * u;
       }
       if (sl == 0 && col < vdim) out[(t0 + base + tt) * ((int64_t)heads * vdim) + h * vdim + col] = g * rq_ + kq * u;
     }
@@ -187,8 +205,8 @@ extern "C" int aphro_gated_delta_scan(float* out, const void* q, int64_t q_strid
                                       int64_t v_stride, const void* b, int64_t b_stride, const void* a, int64_t a_stride,
                                       const float* a_log, const float* dt_bias, float* state, const int32_t* slot_of_seq,
                                       int num_slots, const int32_t* q_start, const int32_t* q_len, const int32_t* ctx_len,
-                                      int num_seqs, int64_t num_tokens, int heads, int kv_heads, int dim, int vdim, float q_scale,
-                                      float norm_eps, int max_q_len, int dtype, void* stream) {
+                                      int num_seqs, int64_t num_tokens, int heads, int kv_heads, int dim, int vdim, int channel_decay,
+                                      float q_scale, float norm_eps, int max_q_len, int dtype, void* stream) {
   if (num_tokens == 0 || num_seqs == 0) return APHRO_OK;
   APHRO_CHECK(out && q && k && v && b && a && a_log && dt_bias && state && slot_of_seq && q_start && q_len && ctx_len,
               "gated_delta_scan: null argument");
@@ -196,14 +214,19 @@ extern "C" int aphro_gated_delta_scan(float* out, const void* q, int64_t q_strid
                   vdim <= 16 * 65535 && num_slots > 0,
               "gated_delta_scan: heads %d over %d key heads, dim %d (<= 256), vdim %d", heads, kv_heads, dim, vdim);
   APHRO_CHECK(q_stride >= (int64_t)kv_heads * dim && k_stride >= (int64_t)kv_heads * dim && v_stride >= (int64_t)heads * vdim &&
-                  b_stride >= heads && a_stride >= heads, "gated_delta_scan: row strides smaller than the rows");
+                  b_stride >= heads && a_stride >= (channel_decay ? (int64_t)heads * dim : (int64_t)heads), "gated_delta_scan: row strides smaller than the rows");
   const bool wide = max_q_len >= 32;
   const int tw = wide ? 16 : 64;
   const dim3 grid((unsigned)num_seqs, (unsigned)heads, (unsigned)((vdim + tw - 1) / tw));
-#define GDR_LAUNCH(DPT, SLOG)                                                                                                  \
-  hipLaunchKernelGGL((gated_delta_scan_kernel<T, DPT, SLOG>), grid, dim3(256), 0, (hipStream_t)stream, out, (const S*)q, q_stride, \
+#define GDR_LAUNCH1(DPT, SLOG, CHANNEL)                                                                                                \
+  hipLaunchKernelGGL((gated_delta_scan_kernel<T, DPT, SLOG, CHANNEL>), grid, dim3(256), 0, (hipStream_t)stream, out, (const S*)q, q_stride, \
                      (const S*)k, k_stride, (const S*)v, v_stride, (const S*)b, b_stride, (const S*)a, a_stride, a_log, dt_bias,  \
                      state, slot_of_seq, num_slots, q_start, q_len, ctx_len, heads, kv_heads, dim, vdim, q_scale, norm_eps)
+#define GDR_LAUNCH(DPT, SLOG)                             \
+  do {                                                    \
+    if (channel_decay) GDR_LAUNCH1(DPT, SLOG, true);      \
+    else GDR_LAUNCH1(DPT, SLOG, false);                   \
+  } while (0)
   MIX_DISPATCH_DTYPE(dtype, {
     typedef typename T::storage S;
     if (wide) {
@@ -216,6 +239,7 @@ extern "C" int aphro_gated_delta_scan(float* out, const void* q, int64_t q_strid
     else GDR_LAUNCH(64, 2);
   });
 #undef GDR_LAUNCH
+#undef GDR_LAUNCH1
   APHRO_LAUNCH_CHECK();
   return APHRO_OK;
 }

@@ -51,6 +51,7 @@ __device__ __forceinline__ float gelu_tanh_f(float z) {
   const float u = 0.7978845608028654f * (z + 0.044715f * z * z * z);
   return 0.5f * z * (1.0f + tanhf(u));
 }
+__device__ __forceinline__ float softplus_f(float z) { return z > 20.f ? z : log1pf(expf(z)); }
 // log(sigmoid(z)) without overflow on either side
 __device__ __forceinline__ float log_sigmoid_f(float z) {
   return fminf(z, 0.f) - log1pf(expf(-fabsf(z)));

@@ -21,13 +21,18 @@ namespace aphro {
 
 template <typename T>
 __global__ void embed_scale_kernel(float* __restrict__ residual, const typename T::storage* __restrict__ table,
-                                   const int64_t* __restrict__ ids, int width, int64_t vocab, float scale) {
+                                   const int64_t* __restrict__ ids, int width, int64_t vocab, float scale,
+                                   typename T::storage* __restrict__ copy) {
   const int64_t t = blockIdx.x;
   int64_t id = ids[t];
   if (id < 0 || id >= vocab) id = 0;           // the host validates ids; never read outside the table
   const typename T::storage* row = table + id * (int64_t)width;
   float* o = residual + t * (int64_t)width;
-  for (int i = threadIdx.x; i < width; i += blockDim.x) o[i] = T::to_f32(row[i]) * scale;
+  for (int i = threadIdx.x; i < width; i += blockDim.x) {
+    const float x = T::to_f32(row[i]) * scale;
+    o[i] = x;
+    if (copy) copy[t * (int64_t)width + i] = T::from_f32(x);
+  }
 }
 
 // mean and 1/sqrt(var + eps) of the row held in LDS (fp32), variance as the mean of squared deviations
@@ -233,6 +238,116 @@ __global__ void gated_group_rms_norm_kernel(typename T::storage* __restrict__ ou
   }
 }
 
+// x += y / rms(y) * w, then out = x / rms(x) * pre_w, or -- without pre_w -- x itself.  One workgroup per row.
+template <typename T>
+__global__ void residual_post_rms_norm_kernel(float* __restrict__ residual, const typename T::storage* __restrict__ y, int64_t y_stride,
+                                              const typename T::storage* __restrict__ post_w, const typename T::storage* __restrict__ pre_w,
+                                              typename T::storage* __restrict__ out, int width, float eps) {
+  __shared__ float red[16];
+  const int64_t t = blockIdx.x;
+  float* r = residual + t * (int64_t)width;
+  if (y) {
+    const typename T::storage* yr = y + t * y_stride;
+    float ss = 0.f;
+    for (int i = threadIdx.x; i < width; i += blockDim.x) {
+      const float v = T::to_f32(yr[i]);
+      ss += v * v;
+    }
+    const float rstd = 1.0f / sqrtf(wg_sum(ss, red) / (float)width + eps);
+    for (int i = threadIdx.x; i < width; i += blockDim.x) r[i] += T::to_f32(yr[i]) * rstd * T::to_f32(post_w[i]);
+  }
+  if (out == nullptr) return;                              // (a thread reads below only what it has written itself)
+  float f = 1.f;
+  if (pre_w) {
+    float ss = 0.f;
+    for (int i = threadIdx.x; i < width; i += blockDim.x) ss += r[i] * r[i];
+    f = 1.0f / sqrtf(wg_sum(ss, red) / (float)width + eps);
+  }
+  typename T::storage* o = out + t * (int64_t)width;
+  for (int i = threadIdx.x; i < width; i += blockDim.x) o[i] = T::from_f32(pre_w ? r[i] * f * T::to_f32(pre_w[i]) : r[i]);
+}
+
+template <typename T>
+__global__ void residual_post_rms_norm_vec8_kernel(float* __restrict__ residual, const typename T::storage* __restrict__ y,
+                                                   int64_t y_stride, const typename T::storage* __restrict__ post_w,
+                                                   const typename T::storage* __restrict__ pre_w, typename T::storage* __restrict__ out,
+                                                   int width, float eps) {
+  __shared__ float red[16];
+  const int64_t t = blockIdx.x;
+  const int i0 = threadIdx.x * 8;
+  const bool act = i0 < width;
+  const int ia = act ? i0 : 0;
+  float* r = residual + t * (int64_t)width;
+  float rv[8], x[8], w[8], pw[8];
+  load8<Float>(r + ia, rv);
+  if (y) {
+    load8<T>(y + t * y_stride + ia, x);
+    load8<T>(post_w + ia, w);
+  }
+  if (pre_w) load8<T>(pre_w + ia, pw);
+  if (y) {
+    float ss = 0.f;
+#pragma unroll
+    for (int j = 0; j < 8; ++j) ss += act ? x[j] * x[j] : 0.f;
+    const float rstd = 1.0f / sqrtf(wg_sum(ss, red) / (float)width + eps);
+#pragma unroll
+    for (int j = 0; j < 8; ++j) rv[j] += x[j] * rstd * w[j];
+    if (act) store8<Float>(r + i0, rv);
+  }
+  if (out == nullptr) return;
+  if (pre_w) {
+    float ss = 0.f;
+#pragma unroll
+    for (int j = 0; j < 8; ++j) ss += act ? rv[j] * rv[j] : 0.f;
+    const float f = 1.0f / sqrtf(wg_sum(ss, red) / (float)width + eps);
+#pragma unroll
+    for (int j = 0; j < 8; ++j) rv[j] *= f * pw[j];
+  }
+  if (act) store8<T>(out + t * (int64_t)width + i0, rv);
+}
+
+// out = out_scale * z / rms(z over a part of the row) * weight,  z = x * silu(gate): the gate comes before the norm.
+// One workgroup per (row, part); a thread keeps 8 numbers per step of the block in registers (VEC), or reads twice.
+template <typename T, bool VEC>
+__global__ __launch_bounds__(1024) void silu_gate_part_rms_norm_kernel(typename T::storage* __restrict__ out, int64_t out_stride,
+                                                                       const float* __restrict__ x,
+                                                                       const typename T::storage* __restrict__ gate, int64_t gate_stride,
+                                                                       const typename T::storage* __restrict__ weight, int n, int part,
+                                                                       float eps, float out_scale) {
+  __shared__ float red[16];
+  const int64_t t = blockIdx.x;
+  const int p0 = blockIdx.y * part;
+  const float* xr = x + t * (int64_t)n + p0;
+  const typename T::storage* gr = gate + t * gate_stride + p0;
+  typename T::storage* o = out + t * out_stride + p0;
+  float ss = 0.f;
+  if constexpr (VEC) {
+    const int i0 = threadIdx.x * 8;
+    const bool act = i0 < part;
+    float z[8], g[8], w[8];
+    load8<Float>(xr + (act ? i0 : 0), z);
+    load8<T>(gr + (act ? i0 : 0), g);
+    load8<T>(weight + p0 + (act ? i0 : 0), w);
+#pragma unroll
+    for (int j = 0; j < 8; ++j) {
+      z[j] *= silu_f(g[j]);
+      ss += act ? z[j] * z[j] : 0.f;
+    }
+    const float f = out_scale / sqrtf(wg_sum(ss, red) / (float)part + eps);
+#pragma unroll
+    for (int j = 0; j < 8; ++j) z[j] *= f * w[j];
+    if (act) store8<T>(o + i0, z);
+  } else {
+    for (int i = threadIdx.x; i < part; i += blockDim.x) {
+      const float z = xr[i] * silu_f(T::to_f32(gr[i]));
+      ss += z * z;
+    }
+    const float f = out_scale / sqrtf(wg_sum(ss, red) / (float)part + eps);
+    for (int i = threadIdx.x; i < part; i += blockDim.x)
+      o[i] = T::from_f32(xr[i] * silu_f(T::to_f32(gr[i])) * f * T::to_f32(weight[p0 + i]));
+  }
+}
+
 static int block_for(int width) { return width >= 1024 ? 256 : (width > 256 ? 128 : 64); }
 
 }  // namespace aphro
@@ -240,12 +355,12 @@ static int block_for(int width) { return width >= 1024 ? 256 : (width > 256 ? 12
 using namespace aphro;
 
 extern "C" int aphro_embed_scale_f32(float* residual, const void* table, const int64_t* ids, int64_t num_tokens, int width,
-                                     int64_t vocab, float scale, int dtype, void* stream) {
+                                     int64_t vocab, float scale, void* copy, int dtype, void* stream) {
   if (num_tokens == 0) return APHRO_OK;
   APHRO_CHECK(residual && table && ids && num_tokens > 0 && width > 0 && vocab > 0, "embed_scale: bad arguments");
   MIX_DISPATCH_DTYPE(dtype, hipLaunchKernelGGL((embed_scale_kernel<T>), dim3((unsigned)num_tokens), dim3(block_for(width)),
                                                0, (hipStream_t)stream, residual, (const typename T::storage*)table, ids, width,
-                                               vocab, scale));
+                                               vocab, scale, (typename T::storage*)copy));
   APHRO_LAUNCH_CHECK();
   return APHRO_OK;
 }
@@ -325,6 +440,50 @@ extern "C" int aphro_gated_group_rms_norm(void* out, int64_t out_stride, const f
     hipLaunchKernelGGL((gated_group_rms_norm_kernel<T>), dim3((unsigned)num_tokens), dim3(block_for(group)), 0,
                        (hipStream_t)stream, (S*)out, out_stride, x, (const S*)weight, (const S*)gate, gate_stride, n, group,
                        eps, out_scale);
+  });
+  APHRO_LAUNCH_CHECK();
+  return APHRO_OK;
+}
+
+extern "C" int aphro_residual_post_rms_norm(float* residual, const void* y, int64_t y_stride, const void* post_w, const void* pre_w,
+                                            void* out, int64_t num_tokens, int width, float eps, int dtype, void* stream) {
+  if (num_tokens == 0) return APHRO_OK;
+  APHRO_CHECK(residual && num_tokens > 0 && width > 0, "residual_post_rms_norm: bad sizes (width %d)", width);
+  APHRO_CHECK(!y || (post_w && y_stride >= width), "residual_post_rms_norm: y needs post_w and a row stride >= width");
+  APHRO_CHECK(y || out, "residual_post_rms_norm: nothing to do");
+  const auto al16 = [](const void* ptr) { return ((uintptr_t)ptr & 15) == 0; };
+  const bool vec = (width & 7) == 0 && width <= 8192 && (y_stride & 7) == 0 && al16(residual) && al16(y) && al16(post_w) && al16(pre_w) && al16(out);
+  MIX_DISPATCH_DTYPE(dtype, {
+    typedef typename T::storage S;
+    if (vec)
+      hipLaunchKernelGGL((residual_post_rms_norm_vec8_kernel<T>), dim3((unsigned)num_tokens), dim3(((width / 8) + 63) / 64 * 64), 0,
+                         (hipStream_t)stream, residual, (const S*)y, y_stride, (const S*)post_w, (const S*)pre_w, (S*)out, width, eps);
+    else
+      hipLaunchKernelGGL((residual_post_rms_norm_kernel<T>), dim3((unsigned)num_tokens), dim3(block_for(width)), 0, (hipStream_t)stream,
+                         residual, (const S*)y, y_stride, (const S*)post_w, (const S*)pre_w, (S*)out, width, eps);
+  });
+  APHRO_LAUNCH_CHECK();
+  return APHRO_OK;
+}
+
+extern "C" int aphro_silu_gate_part_rms_norm(void* out, int64_t out_stride, const float* x, const void* gate, int64_t gate_stride,
+                                             const void* weight, int64_t num_tokens, int n, int part, float eps, float out_scale,
+                                             int dtype, void* stream) {
+  if (num_tokens == 0) return APHRO_OK;
+  APHRO_CHECK(out && x && gate && weight && n > 0 && part > 0 && n % part == 0 && n / part <= 65535 && out_stride >= n && gate_stride >= n,
+              "silu_gate_part_rms_norm: bad arguments (n %d part %d)", n, part);
+  const auto al16 = [](const void* ptr) { return ((uintptr_t)ptr & 15) == 0; };
+  const bool vec = (part & 7) == 0 && part <= 8192 && (n & 7) == 0 && (gate_stride & 7) == 0 && (out_stride & 7) == 0 && al16(x) &&
+                   al16(gate) && al16(weight) && al16(out);
+  const dim3 grid((unsigned)num_tokens, (unsigned)(n / part));
+  MIX_DISPATCH_DTYPE(dtype, {
+    typedef typename T::storage S;
+    if (vec)
+      hipLaunchKernelGGL((silu_gate_part_rms_norm_kernel<T, true>), grid, dim3((part / 8 + 63) / 64 * 64), 0, (hipStream_t)stream, (S*)out,
+                         out_stride, x, (const S*)gate, gate_stride, (const S*)weight, n, part, eps, out_scale);
+    else
+      hipLaunchKernelGGL((silu_gate_part_rms_norm_kernel<T, false>), grid, dim3(block_for(part)), 0, (hipStream_t)stream, (S*)out, out_stride,
+                         x, (const S*)gate, gate_stride, (const S*)weight, n, part, eps, out_scale);
   });
   APHRO_LAUNCH_CHECK();
   return APHRO_OK;

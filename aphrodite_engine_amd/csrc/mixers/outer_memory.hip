@@ -5,6 +5,8 @@
 //   mode 0, decay linear attention: q, k, v through silu, a_t = a fixed per-head decay, b_t = 1.
 //   mode 1, mLSTM: exponential input gate and sigmoid forget gate in log space under a running maximum m (which starts at
 //   ZERO), a normaliser vector n that follows the same recurrence with k alone, and the guarded division of the output.
+//   mode 2, selective state space (Mamba-2): dt_t = softplus(raw + dt_bias), a_t = exp(-exp(A_log) dt_t), b_t = dt_t per head;
+//   keys and queries (that literature's B and C) are shared by groups of neighbouring heads; o_t gains D v_t.
 // State, gates, decays and the accumulation are fp32 whatever the activations' storage.
 //
 // Work split: a workgroup of 256 threads owns 64 (or, for prompt portions, 16) value columns of one (segment, head): thread
@@ -26,7 +28,8 @@ __global__ __launch_bounds__(256) void outer_memory_scan_kernel(
     float* __restrict__ state_s, float* __restrict__ state_n, float* __restrict__ state_m,
     const int32_t* __restrict__ slot_of_seq, int num_slots, const int32_t* __restrict__ q_start,
     const int32_t* __restrict__ q_len, const int32_t* __restrict__ ctx_len, int heads, int dim, int vdim,
-    const float* __restrict__ decay, float q_scale, float gate_cap) {
+    const float* __restrict__ decay, float q_scale, float gate_cap, int qk_heads, const float* __restrict__ a_log,
+    const float* __restrict__ dt_bias, const float* __restrict__ skip) {
   constexpr int NS = 1 << SLOG;        // slices of the key dimension = lanes that share a column
   constexpr int TW = 256 >> SLOG;      // value columns per workgroup
   constexpr int DP = NS * DPT;
@@ -37,6 +40,7 @@ __global__ __launch_bounds__(256) void outer_memory_scan_kernel(
   const int s = blockIdx.x, h = blockIdx.y, c0 = blockIdx.z * TW;
   const int ncopy = (vdim + 15) >> 4, copy0 = c0 >> 4;          // n and m are kept once per 16 value columns
   const int tid = threadIdx.x, c = tid >> SLOG, sl = tid & (NS - 1), col = c0 + c;
+  const int hq = MODE == 2 ? h / (heads / qk_heads) : h;    // head of q and k
   const int n = q_len[s];
   const int slot = slot_of_seq[s];
   if (n <= 0 || slot < 0 || slot >= num_slots) return;
@@ -55,6 +59,7 @@ __global__ __launch_bounds__(256) void outer_memory_scan_kernel(
   }
   if (MODE == 1 && !fresh) m = *mptr;
   const float dec = MODE == 0 ? decay[h] : 0.f;
+  const float neg_rate = MODE == 2 ? -expf(a_log[h]) : 0.f, dtb = MODE == 2 ? dt_bias[h] : 0.f, skip_h = MODE == 2 ? skip[h] : 0.f;
 
   // raw q / k / v (and gates) of the next stage travel in registers while the current stage is scanned
   constexpr int NQ = (OMS_CH * DP + 255) / 256, NV = (OMS_CH * TW + 255) / 256;
@@ -66,8 +71,8 @@ __global__ __launch_bounds__(256) void outer_memory_scan_kernel(
       const int idx = tid + 256 * it, tt = idx / DP, r = idx % DP;
       rq[it] = rk[it] = 0.f;
       if (tt < cnt && r < dim) {
-        rq[it] = T::to_f32(q[(t0 + base + tt) * q_stride + h * dim + r]);
-        rk[it] = T::to_f32(k[(t0 + base + tt) * k_stride + h * dim + r]);
+        rq[it] = T::to_f32(q[(t0 + base + tt) * q_stride + hq * dim + r]);
+        rk[it] = T::to_f32(k[(t0 + base + tt) * k_stride + hq * dim + r]);
       }
     }
 #pragma unroll
@@ -79,6 +84,7 @@ __global__ __launch_bounds__(256) void outer_memory_scan_kernel(
       rgi = T::to_f32(gate_i[(t0 + base + tid) * gate_stride + h]);
       rgf = T::to_f32(gate_f[(t0 + base + tid) * gate_stride + h]);
     }
+    if (MODE == 2 && tid < cnt) rgi = T::to_f32(gate_i[(t0 + base + tid) * gate_stride + h]);
   };
   fetch(0);
   for (int base = 0; base < n; base += OMS_CH) {
@@ -88,7 +94,7 @@ __global__ __launch_bounds__(256) void outer_memory_scan_kernel(
     for (int it = 0; it < NQ; ++it) {
       const int idx = tid + 256 * it, tt = idx / DP, r = idx % DP;
       if (tt < OMS_CH) {
-        qs[tt][r] = MODE == 0 ? silu_f(rq[it]) : rq[it] * q_scale;
+        qs[tt][r] = MODE == 0 ? silu_f(rq[it]) : MODE == 1 ? rq[it] * q_scale : rq[it];
         ks[tt][r] = MODE == 0 ? silu_f(rk[it]) : rk[it];
       }
     }
@@ -96,6 +102,11 @@ __global__ __launch_bounds__(256) void outer_memory_scan_kernel(
     for (int it = 0; it < NV; ++it) {
       const int idx = tid + 256 * it;
       if (idx < OMS_CH * TW) vs[idx / TW][idx % TW] = MODE == 0 ? silu_f(rv[it]) : rv[it];
+    }
+    if (MODE == 2 && tid < cnt) {
+      const float dt = softplus_f(rgi + dtb);
+      a_s[tid] = expf(neg_rate * dt);
+      b_s[tid] = dt;
     }
     if (MODE == 1 && tid < 64) {
       float gi = 0.f, gf = 0.f;
@@ -124,8 +135,8 @@ __global__ __launch_bounds__(256) void outer_memory_scan_kernel(
     if (base + OMS_CH < n) fetch(base + OMS_CH);
 #pragma unroll 4
     for (int tt = 0; tt < cnt; ++tt) {
-      const float a = MODE == 1 ? a_s[tt] : dec;
-      const float b = MODE == 1 ? b_s[tt] : 1.0f;
+      const float a = MODE != 0 ? a_s[tt] : dec;
+      const float b = MODE != 0 ? b_s[tt] : 1.0f;
       const float vv = vs[tt][c] * b;
       float part[4] = {0.f, 0.f, 0.f, 0.f}, npart[4] = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
@@ -149,6 +160,7 @@ __global__ __launch_bounds__(256) void outer_memory_scan_kernel(
         pn = group_sum<SLOG>(pn);
         po = po / (fmaxf(fabsf(pn), em_s[tt]) + 1e-6f);
       }
+      if (MODE == 2) po += skip_h * vs[tt][c];
       if (sl == 0 && col < vdim) out[(t0 + base + tt) * ((int64_t)heads * vdim) + h * vdim + col] = po;
     }
   }
@@ -172,16 +184,18 @@ extern "C" int aphro_outer_memory_scan(float* out, const void* q, int64_t q_stri
                                        int64_t gate_stride, float* state_s, float* state_n, float* state_m,
                                        const int32_t* slot_of_seq, int num_slots, const int32_t* q_start, const int32_t* q_len,
                                        const int32_t* ctx_len, int num_seqs, int64_t num_tokens, int heads, int dim, int vdim,
-                                       int mode, const float* decay, float q_scale, float gate_cap, int max_q_len, int dtype,
+                                       int mode, const float* decay, float q_scale, float gate_cap, int qk_heads,
+                                       const float* a_log, const float* dt_bias, const float* skip, int max_q_len, int dtype,
                                        void* stream) {
   if (num_tokens == 0 || num_seqs == 0) return APHRO_OK;
   APHRO_CHECK(out && q && k && v && state_s && slot_of_seq && q_start && q_len && ctx_len, "outer_memory_scan: null argument");
-  APHRO_CHECK(mode == 0 || mode == 1, "outer_memory_scan: mode %d", mode);
-  APHRO_CHECK(mode == 0 ? decay != nullptr : (gate_i && gate_f && state_n && state_m && gate_cap > 0.f && gate_stride >= heads),
+  APHRO_CHECK(mode >= 0 && mode <= 2, "outer_memory_scan: mode %d", mode);
+  APHRO_CHECK(qk_heads > 0 && heads % qk_heads == 0 && (mode == 2 || qk_heads == heads), "outer_memory_scan: %d heads over %d query/key heads", heads, qk_heads);
+  APHRO_CHECK(mode == 0 ? decay != nullptr : mode == 2 ? (gate_i && a_log && dt_bias && skip && gate_stride >= heads) : (gate_i && gate_f && state_n && state_m && gate_cap > 0.f && gate_stride >= heads),
               "outer_memory_scan: mode %d lacks its gate arguments", mode);
   APHRO_CHECK(heads > 0 && heads <= 65535 && dim > 0 && dim <= 256 && vdim > 0 && vdim <= 64 * 65535 && num_slots > 0 && num_seqs > 0,
               "outer_memory_scan: heads %d dim %d (<= 256) vdim %d", heads, dim, vdim);
-  APHRO_CHECK(q_stride >= (int64_t)heads * dim && k_stride >= (int64_t)heads * dim && v_stride >= (int64_t)heads * vdim,
+  APHRO_CHECK(q_stride >= (int64_t)qk_heads * dim && k_stride >= (int64_t)qk_heads * dim && v_stride >= (int64_t)heads * vdim,
               "outer_memory_scan: row strides smaller than the rows");
   // Prompt portions: 16 lanes per value column (16 columns per workgroup), so that a long sequential scan spreads over four
   // times as many waves with a quarter of the work per token and lane.  Single tokens: 4 lanes per column (64 columns per
@@ -193,7 +207,7 @@ extern "C" int aphro_outer_memory_scan(float* out, const void* q, int64_t q_stri
   hipLaunchKernelGGL((outer_memory_scan_kernel<T, MODE, DPT, SLOG>), grid, dim3(256), 0, (hipStream_t)stream, out, (const S*)q, \
                      q_stride, (const S*)k, k_stride, (const S*)v, v_stride, (const S*)gate_i, (const S*)gate_f, gate_stride, \
                      state_s, state_n, state_m, slot_of_seq, num_slots, q_start, q_len, ctx_len, heads, dim, vdim, decay,     \
-                     q_scale, gate_cap)
+                     q_scale, gate_cap, qk_heads, a_log, dt_bias, skip)
 #define OMS_BY_DIM(MODE)                               \
   do {                                                 \
     if (wide) {                                        \
@@ -210,7 +224,8 @@ extern "C" int aphro_outer_memory_scan(float* out, const void* q, int64_t q_stri
   MIX_DISPATCH_DTYPE(dtype, {
     typedef typename T::storage S;
     if (mode == 0) OMS_BY_DIM(0);
-    else OMS_BY_DIM(1);
+    else if (mode == 1) OMS_BY_DIM(1);
+    else OMS_BY_DIM(2);
   });
 #undef OMS_BY_DIM
 #undef OMS_LAUNCH

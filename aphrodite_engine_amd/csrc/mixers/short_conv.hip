@@ -1,5 +1,5 @@
 // Short causal convolution over time on every channel of a projection's output, for a batch of segments:
-//   y_t[c] = sum_j w[c, j] * u_(t - taps + 1 + j)[c],   zeros before the sequence's start.
+//   y_t[c] = sum_j w[c, j] * u_(t - taps + 1 + j)[c]  (+ b[c]),   zeros before the sequence's start.
 // The taps - 1 inputs that precede a segment come from the request's state slot, which afterwards holds the last taps - 1
 // inputs of the sequence.  A segment that starts a sequence never reads its slot, and no input older than the sequence's
 // start is read from it either, so a slot taken over from another request needs no clearing.
@@ -18,7 +18,8 @@ __global__ void short_conv_kernel(typename T::storage* __restrict__ q_out, int64
                                   typename T::storage* __restrict__ k_cache, typename T::storage* __restrict__ v_cache,
                                   const int64_t* __restrict__ cache_slots, int64_t num_cache_slots,
                                   const typename T::storage* __restrict__ u, int64_t u_stride,
-                                  const typename T::storage* __restrict__ w, const typename T::storage* __restrict__ state,
+                                  const typename T::storage* __restrict__ w, const typename T::storage* __restrict__ bias,
+                                  const typename T::storage* __restrict__ state,
                                   const int32_t* __restrict__ state_slots, const int32_t* __restrict__ q_start,
                                   const int32_t* __restrict__ ctx_len, const int32_t* __restrict__ seq_of_token, int cq, int ck,
                                   int cv, int taps, int act) {
@@ -29,7 +30,7 @@ __global__ void short_conv_kernel(typename T::storage* __restrict__ q_out, int64
   const int s = seq_of_token[t];
   const int r = (int)t - q_start[s], ctx = ctx_len[s];
   const typename T::storage* st = state ? state + ((int64_t)state_slots[s] * (taps - 1)) * C + c : nullptr;
-  float acc = 0.f;
+  float acc = bias ? T::to_f32(bias[c]) : 0.f;
   for (int j = 0; j < taps; ++j) {
     const int i = r - taps + 1 + j;            // row of the segment, negative: before it
     float x = 0.f;
@@ -84,6 +85,7 @@ __global__ __launch_bounds__(256) void short_conv_vec8_kernel(
     typename T::storage* __restrict__ q_out, int64_t q_out_stride, typename T::storage* __restrict__ k_cache,
     typename T::storage* __restrict__ v_cache, const int64_t* __restrict__ cache_slots, int64_t num_cache_slots,
     const typename T::storage* __restrict__ u, int64_t u_stride, const typename T::storage* __restrict__ w,
+    const typename T::storage* __restrict__ bias,
     const typename T::storage* __restrict__ state, const int32_t* __restrict__ state_slots, const int32_t* __restrict__ q_start,
     const int32_t* __restrict__ ctx_len, const int32_t* __restrict__ seq_of_token, int64_t num_tokens, int cq, int ck, int cv,
     int act) {
@@ -101,6 +103,8 @@ __global__ __launch_bounds__(256) void short_conv_vec8_kernel(
 #pragma unroll
       for (int j = 0; j < TAPS; ++j) wv[j][i] = flat[i * TAPS + j];
   }
+  float bv[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
+  if (bias) sc_load8<T>(bias + c0, bv);
   float rows[TOK + TAPS - 1][8];
 #pragma unroll
   for (int x = 0; x < TOK + TAPS - 1; ++x) {
@@ -120,7 +124,7 @@ __global__ __launch_bounds__(256) void short_conv_vec8_kernel(
     const int r = (int)t - q_start[s], ctx = ctx_len[s];
     float acc[8];
 #pragma unroll
-    for (int i = 0; i < 8; ++i) acc[i] = 0.f;
+    for (int i = 0; i < 8; ++i) acc[i] = bv[i];
 #pragma unroll
     for (int j = 0; j < TAPS; ++j) {
       const int i0 = r - TAPS + 1 + j;         // row of the segment, negative: before it
@@ -181,7 +185,8 @@ __global__ void short_conv_state_kernel(typename T::storage* __restrict__ state,
 using namespace aphro;
 
 extern "C" int aphro_short_conv(void* q_out, int64_t q_out_stride, void* k_cache, void* v_cache, const int64_t* cache_slots,
-                                int64_t num_cache_slots, const void* u, int64_t u_stride, const void* w, void* state,
+                                int64_t num_cache_slots, const void* u, int64_t u_stride, const void* w, const void* bias,
+                                void* state,
                                 const int32_t* state_slots, const int32_t* q_start, const int32_t* q_len,
                                 const int32_t* ctx_len, const int32_t* seq_of_token, int64_t num_tokens, int num_seqs, int cq,
                                 int ck, int cv, int taps, int act, int dtype, void* stream) {
@@ -198,12 +203,12 @@ extern "C" int aphro_short_conv(void* q_out, int64_t q_out_stride, void* k_cache
   APHRO_CHECK(num_tokens <= 0x7fffffff && (C + 255) / 256 <= 65535, "short_conv: too large");
   const auto al16 = [](const void* ptr) { return ((uintptr_t)ptr & 15) == 0; };
   const bool vec = taps >= 2 && taps <= 4 && (cq & 7) == 0 && (ck & 7) == 0 && (cv & 7) == 0 && (u_stride & 7) == 0 &&
-                   (q_out_stride & 7) == 0 && al16(u) && al16(w) && al16(q_out) && al16(k_cache) && al16(v_cache) && al16(state);
+                   (q_out_stride & 7) == 0 && al16(u) && al16(w) && al16(bias) && al16(q_out) && al16(k_cache) && al16(v_cache) && al16(state);
   constexpr int TOK = 4;
 #define SC_VEC(TAPS)                                                                                                           \
   hipLaunchKernelGGL((short_conv_vec8_kernel<T, TAPS, TOK>), dim3((unsigned)((num_tokens + TOK - 1) / TOK), (unsigned)((C / 8 + 255) / 256)), \
                      dim3(C / 8 >= 256 ? 256 : (C / 8 + 63) / 64 * 64), 0, (hipStream_t)stream, (S*)q_out, q_out_stride, (S*)k_cache,     \
-                     (S*)v_cache, cache_slots, num_cache_slots, (const S*)u, u_stride, (const S*)w, (const S*)state, state_slots,        \
+                     (S*)v_cache, cache_slots, num_cache_slots, (const S*)u, u_stride, (const S*)w, (const S*)bias, (const S*)state, state_slots, \
                      q_start, ctx_len, seq_of_token, num_tokens, cq, ck, cv, act)
   MIX_DISPATCH_DTYPE(dtype, {
     typedef typename T::storage S;
@@ -213,7 +218,7 @@ extern "C" int aphro_short_conv(void* q_out, int64_t q_out_stride, void* k_cache
     else
     hipLaunchKernelGGL((short_conv_kernel<T>), dim3((unsigned)num_tokens, (unsigned)((C + 255) / 256)), dim3(256), 0,
                        (hipStream_t)stream, (S*)q_out, q_out_stride, (S*)k_cache, (S*)v_cache, cache_slots, num_cache_slots,
-                       (const S*)u, u_stride, (const S*)w, (const S*)state, state_slots, q_start, ctx_len, seq_of_token, cq, ck,
+                       (const S*)u, u_stride, (const S*)w, (const S*)bias, (const S*)state, state_slots, q_start, ctx_len, seq_of_token, cq, ck,
                        cv, taps, act);
     if (taps > 1)
       hipLaunchKernelGGL((short_conv_state_kernel<T>), dim3((unsigned)num_seqs, (unsigned)((C + 255) / 256)), dim3(256), 0,

@@ -298,6 +298,17 @@ def iter_safetensors(model_dir: str) -> Iterator[Tuple[str, torch.Tensor]]:
                 yield name, f.get_tensor(name)
 
 
+def safetensors_shapes(model_dir: str) -> Dict[str, Tuple[int, ...]]:
+    """name -> shape of every tensor of the checkpoint, from the files' headers (for the sizes a config.json leaves to them)."""
+    from safetensors import safe_open
+    shapes: Dict[str, Tuple[int, ...]] = {}
+    for path in sorted(glob.glob(os.path.join(model_dir, "*.safetensors"))):
+        with safe_open(path, framework="pt", device="cpu") as f:
+            for name in f.keys():
+                shapes[name] = tuple(f.get_slice(name).get_shape())
+    return shapes
+
+
 # --------------------------------------------------------------------------------------------------
 # Llama name mapping
 # --------------------------------------------------------------------------------------------------

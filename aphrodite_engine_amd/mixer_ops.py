@@ -11,7 +11,7 @@ from ._lib import check_mixers as check
 
 _DT = {torch.bfloat16: _lib.BF16, torch.float32: _lib.F32}
 ACT_SILU, ACT_GELU_TANH = 0, 1
-MEMORY_DECAY, MEMORY_MLSTM = 0, 1
+MEMORY_DECAY, MEMORY_MLSTM, MEMORY_STATE_SPACE = 0, 1, 2
 
 
 def _stream() -> int:
@@ -54,17 +54,21 @@ def _i32(t: torch.Tensor, n: int, what: str) -> None:
     _need(t.dtype == torch.int32 and t.is_contiguous() and t.numel() == n, f"{what}: int32 [{n}] expected")
 
 
-def embed_scale(table: torch.Tensor, ids: torch.Tensor, scale: float, out: Optional[torch.Tensor] = None) -> torch.Tensor:
-    """fp32 residual rows ``table[ids] * scale`` (into ``out`` fp32 [T, width] if given)."""
-    _cuda(table, ids, out)
+def embed_scale(table: torch.Tensor, ids: torch.Tensor, scale: float, out: Optional[torch.Tensor] = None,
+                copy: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """fp32 residual rows ``table[ids] * scale`` (into ``out`` fp32 [T, width] if given); ``copy`` [T, width] of the table's dtype
+    takes the same rows rounded."""
+    _cuda(table, ids, out, copy)
     _need(table.dim() == 2 and table.is_contiguous() and ids.dtype == torch.int64 and ids.dim() == 1 and ids.is_contiguous(),
           "embed_scale: table [vocab, width] contiguous, ids int64 [T]")
     if out is None:
         out = torch.empty(ids.shape[0], table.shape[1], dtype=torch.float32, device=table.device)
     _need(out.dtype == torch.float32 and out.is_contiguous() and out.shape == (ids.shape[0], table.shape[1]),
           "embed_scale: out fp32 [T, width], contiguous")
+    _need(copy is None or (copy.dtype == table.dtype and copy.is_contiguous() and copy.shape == out.shape),
+          "embed_scale: copy [T, width] of the table's dtype")
     check(_lib.mixers_lib().aphro_embed_scale_f32(out.data_ptr(), table.data_ptr(), ids.data_ptr(), ids.shape[0],
-                                                  table.shape[1], table.shape[0], float(scale), _dt(table), _stream()),
+                                                  table.shape[1], table.shape[0], float(scale), _p(copy), _dt(table), _stream()),
           "embed_scale")
     return out
 
@@ -101,6 +105,44 @@ def residual_layer_norm(residual: torch.Tensor, y: Optional[torch.Tensor] = None
 
 def _dt_of(dtype):
     return _DT.get(dtype)
+
+
+def residual_post_rms_norm(residual: torch.Tensor, y: Optional[torch.Tensor] = None, post: Optional[torch.Tensor] = None,
+                           pre: Optional[torch.Tensor] = None, eps: float = 1e-6, dtype: Optional[torch.dtype] = None,
+                           want_out: bool = True) -> Optional[torch.Tensor]:
+    """``residual += rms_norm(y) * post`` in place (fp32 [T, W]; without ``y`` not), then returns ``rms_norm(residual) * pre`` -- or,
+    without ``pre``, the residual itself -- in the activation dtype (``want_out`` False: nothing)."""
+    T, W = residual.shape
+    _cuda(residual, y, post, pre)
+    _need(residual.dtype == torch.float32 and residual.is_contiguous(), "residual_post_rms_norm: the residual is fp32, contiguous")
+    some = next((t for t in (y, pre) if t is not None), None)
+    adt = dtype or (some.dtype if some is not None else None)
+    _need(adt in _DT, "residual_post_rms_norm: the activation dtype is not given")
+    ys = 0
+    if y is not None:
+        _need(post is not None and y.dtype == adt and y.shape[0] == T, "residual_post_rms_norm: y [T, W] needs its norm's weight")
+        ys = _rows(y, W, "residual_post_rms_norm y")
+    for v in (post, pre):
+        _need(v is None or (v.dtype == adt and v.numel() == W and v.is_contiguous()), "residual_post_rms_norm: vectors [W] of the activation dtype")
+    _need(y is not None or want_out, "residual_post_rms_norm: nothing to do")
+    out = torch.empty(T, W, dtype=adt, device=residual.device) if want_out else None
+    check(_lib.mixers_lib().aphro_residual_post_rms_norm(residual.data_ptr(), _p(y), ys, _p(post), _p(pre), _p(out), T, W, float(eps),
+                                                         _DT[adt], _stream()), "residual_post_rms_norm")
+    return out
+
+
+def silu_gate_part_rms_norm(out: torch.Tensor, x: torch.Tensor, gate: torch.Tensor, weight: torch.Tensor, parts: int, eps: float,
+                            out_scale: float = 1.0) -> None:
+    """out [T, N] (dense rows, any row stride) = out_scale * z / rms(z over its part) * weight, z = x * silu(gate); a row forms
+    ``parts`` equal parts; x fp32 [T, N] contiguous, gate [T, N] and weight [N] of the output dtype."""
+    _cuda(out, x, gate, weight)
+    T, N = x.shape
+    _need(x.dtype == torch.float32 and x.is_contiguous() and parts > 0 and N % parts == 0, "silu_gate_part_rms_norm: x fp32 [T, N], N a multiple of the parts")
+    _need(out.shape == (T, N) and gate.shape == (T, N) and gate.dtype == out.dtype, "silu_gate_part_rms_norm: out and gate [T, N] of one dtype")
+    _need(weight.dtype == out.dtype and weight.numel() == N and weight.is_contiguous(), "silu_gate_part_rms_norm: weight [N]")
+    check(_lib.mixers_lib().aphro_silu_gate_part_rms_norm(
+        out.data_ptr(), _rows(out, N, "silu_gate_part_rms_norm out"), x.data_ptr(), gate.data_ptr(), _rows(gate, N, "silu_gate_part_rms_norm gate"),
+        weight.data_ptr(), T, N, N // parts, float(eps), float(out_scale), _dt(out), _stream()), "silu_gate_part_rms_norm")
 
 
 def act_and_mul(x: torch.Tensor, act: int) -> torch.Tensor:
@@ -151,14 +193,17 @@ def distance_bias_attention(out: torch.Tensor, q: torch.Tensor, gate: Optional[t
                             v_cache: torch.Tensor, block_tables: torch.Tensor, q_start: torch.Tensor, q_len: torch.Tensor,
                             ctx_len: torch.Tensor, seq_of_token: torch.Tensor, q_len_range, heads: int, scale: float,
                             bias_lut: Optional[torch.Tensor], temp_coef: float = 0.0, temp_every: int = 1,
-                            out_scale: float = 1.0, max_kv_len: int = 0) -> None:
+                            out_scale: float = 1.0, max_kv_len: int = 0, window: int = 0, chunk: int = 0, softcap: float = 0.0,
+                            sink: Optional[torch.Tensor] = None) -> None:
     """Causal attention of a batch of segments over the paged cache, written into ``out`` [T, heads * e] (dense rows, any
-    row stride).  q [T, heads * d]; gate [T, heads] raw (sigmoid inside) or None; bias_lut fp32 [heads, L] indexed by
-    min(distance, L - 1) or None.  ``q_len_range``: (shortest, longest) segment of the batch, known on the host -- it
+    row stride).  q [T, heads * d]; gate raw (sigmoid inside), [T, heads] or elementwise [T, heads * e], or None; bias_lut fp32
+    [heads, L] indexed by min(distance, L - 1) or None.  ``window`` > 0: a row sees itself and the window - 1 tokens before it;
+    ``chunk`` > 0: only keys of its own chunk of positions; ``softcap`` > 0: softcap * tanh(score / softcap) before the bias; ``sink``
+    fp32 [heads]: exp(sink) joins the softmax denominator.  ``q_len_range``: (shortest, longest) segment of the batch, known on the host -- it
     chooses between the matrix-core kernel for prompt portions and the shared-key kernel for single tokens.
     ``max_kv_len``: the longest ctx_len + q_len of the batch (host); given, long key ranges of decoded rows are split over
     several workgroups through a scratch tensor."""
-    _cuda(out, q, gate, k_cache, v_cache, block_tables, q_start, q_len, ctx_len, seq_of_token, bias_lut)
+    _cuda(out, q, gate, k_cache, v_cache, block_tables, q_start, q_len, ctx_len, seq_of_token, bias_lut, sink)
     lo, hi = int(q_len_range[0]), int(q_len_range[1])
     _need(0 < lo <= hi, "distance_bias_attention: q_len_range (shortest, longest)")
     nb, bs, G, d = k_cache.shape
@@ -174,55 +219,69 @@ def distance_bias_attention(out: torch.Tensor, q: torch.Tensor, gate: Optional[t
     _i32(q_len, S, "q_len")
     _i32(ctx_len, S, "ctx_len")
     _i32(seq_of_token, T, "seq_of_token")
-    gs = 0
+    gs = gate_cols = 0
     if gate is not None:
-        _need(gate.dtype == q.dtype and gate.shape[0] == T, "distance_bias_attention: gate [T, heads]")
-        gs = _rows(gate, heads, "gate")
+        _need(gate.dtype == q.dtype and gate.shape[0] == T, "distance_bias_attention: gate [T, heads] or [T, heads * vdim]")
+        gate_cols = 1 if gate.shape[1] != heads else 0
+        gs = _rows(gate, heads * e if gate_cols else heads, "gate")
+    window, chunk, softcap = max(int(window), 0), max(int(chunk), 0), max(float(softcap), 0.0)
+    _need(sink is None or (sink.dtype == torch.float32 and sink.is_contiguous() and sink.numel() == heads),
+          "distance_bias_attention: sink fp32 [heads]")
     L = 0
     if bias_lut is not None:
         _need(bias_lut.dtype == torch.float32 and bias_lut.dim() == 2 and bias_lut.shape[0] == heads and bias_lut.is_contiguous(),
               "distance_bias_attention: bias_lut fp32 [heads, L]")
         L = bias_lut.shape[1]
     ws, ws_n = None, 0
-    if q.dtype == torch.bfloat16 and max_kv_len >= 512 and lo < 8:
+    visible = min([int(max_kv_len)] + [n for n in (window, chunk) if n > 0])
+    if q.dtype == torch.bfloat16 and visible >= 512 and lo < 8:
         ws_n = T * heads * 8 * (2 + e)
         ws = torch.empty(ws_n, dtype=torch.float32, device=q.device)
     check(_lib.mixers_lib().aphro_distance_bias_attention(
         out.data_ptr(), _rows(out, heads * e, "out"), q.data_ptr(), _rows(q, heads * d, "q"), _p(gate), gs, k_cache.data_ptr(),
         v_cache.data_ptr(), block_tables.data_ptr(), block_tables.shape[1], nb, bs, q_start.data_ptr(), q_len.data_ptr(),
         ctx_len.data_ptr(), seq_of_token.data_ptr(), T, S, lo, hi, heads, G, d, e, float(scale), _p(bias_lut), L, float(temp_coef), int(temp_every),
-        float(out_scale), int(max_kv_len), _p(ws), ws_n, _dt(q), _stream()), "distance_bias_attention")
+        float(out_scale), window, chunk, softcap, _p(sink), gate_cols, int(max_kv_len), _p(ws), ws_n, _dt(q), _stream()),
+        "distance_bias_attention")
 
 
 def memory_state_shapes(slots: int, heads: int, dim: int, vdim: int, mode: int):
     """Shapes of the fp32 state tensors of ``outer_memory_scan`` for a pool of ``slots`` requests."""
     tiles = (vdim + 15) // 16
     s = (slots, heads, dim, vdim)
-    return (s, ) if mode == MEMORY_DECAY else (s, (slots, heads, tiles, dim), (slots, heads, tiles))
+    return (s, ) if mode != MEMORY_MLSTM else (s, (slots, heads, tiles, dim), (slots, heads, tiles))
 
 
 def outer_memory_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, state, slot_of_seq: torch.Tensor,
                       q_start: torch.Tensor, q_len: torch.Tensor, ctx_len: torch.Tensor, heads: int, mode: int,
                       decay: Optional[torch.Tensor] = None, gate_i: Optional[torch.Tensor] = None,
                       gate_f: Optional[torch.Tensor] = None, q_scale: float = 1.0, gate_cap: float = 1.0,
-                      max_q_len: int = 1) -> torch.Tensor:
+                      max_q_len: int = 1, qk_heads: int = 0, a_log: Optional[torch.Tensor] = None,
+                      dt_bias: Optional[torch.Tensor] = None, skip: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Scan every segment through its slot's state (updated in place); returns o fp32 [T, heads * vdim].  ``state`` is
     the tuple of tensors shaped by ``memory_state_shapes``.  q, k [T, heads * d], v [T, heads * e]; gates [T, heads] raw.
-    ``max_q_len`` (host: the batch's longest segment) picks the work split: wide for prompt portions, narrow for tokens."""
-    _cuda(q, k, v, slot_of_seq, q_start, q_len, ctx_len, decay, gate_i, gate_f, *state)
+    MEMORY_STATE_SPACE: q and k [T, qk_heads * d] shared by groups of heads, gate_i the raw step sizes, a_log, dt_bias, skip fp32
+    [heads].  ``max_q_len`` (host: the batch's longest segment) picks the work split: wide for prompt portions, narrow for tokens."""
+    _cuda(q, k, v, slot_of_seq, q_start, q_len, ctx_len, decay, gate_i, gate_f, a_log, dt_bias, skip, *state)
+    qk_heads = int(qk_heads) or heads
     T = q.shape[0]
     S = q_start.numel()
     slots, H, d, e = state[0].shape
     _need(H == heads and k.shape[0] == T and v.shape[0] == T and q.dtype == k.dtype == v.dtype, "outer_memory_scan: q, k, v rows / dtype")
     for st, shp in zip(state, memory_state_shapes(slots, heads, d, e, mode)):
         _need(st.dtype == torch.float32 and st.is_contiguous() and tuple(st.shape) == shp, "outer_memory_scan: state tensors")
-    _need(len(state) == (1 if mode == MEMORY_DECAY else 3), "outer_memory_scan: state tuple")
+    _need(len(state) == (3 if mode == MEMORY_MLSTM else 1), "outer_memory_scan: state tuple")
     for t, nm in ((slot_of_seq, "slot_of_seq"), (q_start, "q_start"), (q_len, "q_len"), (ctx_len, "ctx_len")):
         _i32(t, S, nm)
     gs = 0
     if mode == MEMORY_DECAY:
         _need(decay is not None and decay.dtype == torch.float32 and decay.numel() == heads and decay.is_contiguous(),
               "outer_memory_scan: decay fp32 [heads]")
+    elif mode == MEMORY_STATE_SPACE:
+        _need(gate_i is not None and gate_i.dtype == q.dtype and gate_i.shape[0] == T, "outer_memory_scan: step sizes [T, heads]")
+        gs = _rows(gate_i, heads, "gate_i")
+        for t, nm in ((a_log, "a_log"), (dt_bias, "dt_bias"), (skip, "skip")):
+            _need(t is not None and t.dtype == torch.float32 and t.numel() == heads and t.is_contiguous(), f"outer_memory_scan: {nm} fp32 [heads]")
     else:
         _need(gate_i is not None and gate_f is not None and gate_i.dtype == q.dtype == gate_f.dtype
               and gate_i.shape[0] == T and gate_f.shape[0] == T, "outer_memory_scan: gates [T, heads]")
@@ -230,11 +289,12 @@ def outer_memory_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, state, 
         _need(_rows(gate_f, heads, "gate_f") == gs, "outer_memory_scan: the two gates share a row stride")
     out = torch.empty(T, heads * e, dtype=torch.float32, device=q.device)
     check(_lib.mixers_lib().aphro_outer_memory_scan(
-        out.data_ptr(), q.data_ptr(), _rows(q, heads * d, "q"), k.data_ptr(), _rows(k, heads * d, "k"), v.data_ptr(),
+        out.data_ptr(), q.data_ptr(), _rows(q, qk_heads * d, "q"), k.data_ptr(), _rows(k, qk_heads * d, "k"), v.data_ptr(),
         _rows(v, heads * e, "v"), _p(gate_i), _p(gate_f), gs, state[0].data_ptr(),
         state[1].data_ptr() if len(state) > 1 else None, state[2].data_ptr() if len(state) > 2 else None,
         slot_of_seq.data_ptr(), slots, q_start.data_ptr(), q_len.data_ptr(), ctx_len.data_ptr(), S, T, heads, d, e, int(mode),
-        _p(decay), float(q_scale), float(gate_cap), int(max_q_len), _dt(q), _stream()), "outer_memory_scan")
+        _p(decay), float(q_scale), float(gate_cap), qk_heads, _p(a_log), _p(dt_bias), _p(skip), int(max_q_len), _dt(q), _stream()),
+        "outer_memory_scan")
     return out
 
 
@@ -306,16 +366,17 @@ def differential_norm_gate(out: torch.Tensor, a: torch.Tensor, gate: Optional[to
 def short_conv(u: torch.Tensor, w: torch.Tensor, state: Optional[torch.Tensor], state_slots: torch.Tensor, q_start: torch.Tensor,
                q_len: torch.Tensor, ctx_len: torch.Tensor, seq_of_token: torch.Tensor, cq: int, ck: int = 0, cv: int = 0,
                k_cache: Optional[torch.Tensor] = None, v_cache: Optional[torch.Tensor] = None,
-               slot_mapping: Optional[torch.Tensor] = None, act: int = 0) -> Optional[torch.Tensor]:
+               slot_mapping: Optional[torch.Tensor] = None, act: int = 0, bias: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
     """Short causal convolution over time on the channels of u [T, cq + ck + cv] (dense rows, any row stride) with w
-    [channels, taps]; returns the first cq channels [T, cq]; the ck and cv channels go into the paged caches
+    [channels, taps] and an optional bias [channels]; returns the first cq channels [T, cq]; the ck and cv channels go into the paged caches
     (k_cache [blocks, block, ck], v_cache [blocks, block, cv] in any further split of the last axis) at ``slot_mapping``.
     state [slots, taps - 1, channels] holds every request's last inputs and is advanced.  ``act`` 1: silu on the result."""
-    _cuda(u, w, state, state_slots, q_start, q_len, ctx_len, seq_of_token, k_cache, v_cache, slot_mapping)
+    _cuda(u, w, bias, state, state_slots, q_start, q_len, ctx_len, seq_of_token, k_cache, v_cache, slot_mapping)
     C = cq + ck + cv
     T, S = u.shape[0], q_start.numel()
     taps = w.shape[1]
     _need(w.dim() == 2 and w.shape[0] == C and w.is_contiguous() and w.dtype == u.dtype, "short_conv: w [channels, taps]")
+    _need(bias is None or (bias.dtype == u.dtype and bias.numel() == C and bias.is_contiguous()), "short_conv: bias [channels]")
     if taps > 1:
         _need(state is not None and state.dtype == u.dtype and state.dim() == 3 and state.is_contiguous()
               and tuple(state.shape[1:]) == (taps - 1, C), "short_conv: state [slots, taps - 1, channels]")
@@ -333,7 +394,7 @@ def short_conv(u: torch.Tensor, w: torch.Tensor, state: Optional[torch.Tensor], 
     q = torch.empty(T, cq, dtype=u.dtype, device=u.device) if cq else None
     check(_lib.mixers_lib().aphro_short_conv(
         _p(q), cq, _p(k_cache) if ck + cv else None, _p(v_cache) if ck + cv else None, _p(slot_mapping) if ck + cv else None, ncs,
-        u.data_ptr(), _rows(u, C, "short_conv u"), w.data_ptr(), _p(state) if taps > 1 else None, state_slots.data_ptr(),
+        u.data_ptr(), _rows(u, C, "short_conv u"), w.data_ptr(), _p(bias), _p(state) if taps > 1 else None, state_slots.data_ptr(),
         q_start.data_ptr(), q_len.data_ptr(), ctx_len.data_ptr(), seq_of_token.data_ptr(), T, S, cq, ck, cv, taps, int(act), _dt(u),
         _stream()), "short_conv")
     return q
@@ -756,7 +817,8 @@ def gated_delta_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, b: torch
                      max_q_len: int = 1) -> torch.Tensor:
     """Scan every segment through its slot's state S fp32 [slots, heads, dim, vdim] (updated in place) with the gated delta rule;
     returns o fp32 [T, heads * vdim].  q, k [T, kv_heads * dim] (made unit vectors per head inside), v [T, heads * vdim], b and a
-    [T, heads] raw (beta = sigmoid(b), decay = exp(-exp(a_log) softplus(a + dt_bias))); a_log, dt_bias fp32 [heads]."""
+    [T, heads] raw (beta = sigmoid(b), decay = exp(-exp(a_log) softplus(a + dt_bias))); a_log, dt_bias fp32 [heads].  An ``a`` of
+    [T, heads * dim] with dt_bias [heads * dim] means one decay per head and key channel."""
     _cuda(q, k, v, b, a, a_log, dt_bias, state, slot_of_seq, q_start, q_len, ctx_len)
     T, S = q.shape[0], q_start.numel()
     _need(state.dim() == 4 and state.dtype == torch.float32 and state.is_contiguous() and state.shape[1] == heads,
@@ -764,16 +826,18 @@ def gated_delta_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, b: torch
     slots, _, d, e = state.shape
     _need(q.dtype == k.dtype == v.dtype == b.dtype == a.dtype and k.shape[0] == T and v.shape[0] == T and b.shape[0] == T
           and a.shape[0] == T, "gated_delta_scan: q, k, v, b, a rows / dtype")
-    for t, nm in ((a_log, "a_log"), (dt_bias, "dt_bias")):
-        _need(t.dtype == torch.float32 and t.numel() == heads and t.is_contiguous(), f"gated_delta_scan: {nm} fp32 [heads]")
+    channel = a.shape[1] != heads or dt_bias.numel() != heads
+    na = heads * d if channel else heads
+    for t, nm, n in ((a_log, "a_log", heads), (dt_bias, "dt_bias", na)):
+        _need(t.dtype == torch.float32 and t.numel() == n and t.is_contiguous(), f"gated_delta_scan: {nm} fp32 [{n}]")
     for t, nm in ((slot_of_seq, "slot_of_seq"), (q_start, "q_start"), (q_len, "q_len"), (ctx_len, "ctx_len")):
         _i32(t, S, nm)
     out = torch.empty(T, heads * e, dtype=torch.float32, device=q.device)
     check(_lib.mixers_lib().aphro_gated_delta_scan(
         out.data_ptr(), q.data_ptr(), _rows(q, kv_heads * d, "q"), k.data_ptr(), _rows(k, kv_heads * d, "k"), v.data_ptr(),
-        _rows(v, heads * e, "v"), b.data_ptr(), _rows(b, heads, "b"), a.data_ptr(), _rows(a, heads, "a"), a_log.data_ptr(),
+        _rows(v, heads * e, "v"), b.data_ptr(), _rows(b, heads, "b"), a.data_ptr(), _rows(a, na, "a"), a_log.data_ptr(),
         dt_bias.data_ptr(), state.data_ptr(), slot_of_seq.data_ptr(), slots, q_start.data_ptr(), q_len.data_ptr(), ctx_len.data_ptr(),
-        S, T, heads, kv_heads, d, e, float(q_scale), float(norm_eps), int(max_q_len), _dt(q), _stream()), "gated_delta_scan")
+        S, T, heads, kv_heads, d, e, int(channel), float(q_scale), float(norm_eps), int(max_q_len), _dt(q), _stream()), "gated_delta_scan")
     return out
 
 
@@ -805,12 +869,14 @@ ROTARY_HALF, ROTARY_INTERLEAVED = 0, 1
 def rotary_qk_norm_kv_write(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor,
                             slot_mapping: torch.Tensor, q_start: torch.Tensor, ctx_len: torch.Tensor, seq_of_token: torch.Tensor,
                             inv_freq: Optional[torch.Tensor], rot_dims: int, layout: int = ROTARY_HALF, qk_norm: bool = False,
-                            eps: float = 1e-6, v_other: Optional[torch.Tensor] = None, lam: float = 0.0) -> torch.Tensor:
+                            eps: float = 1e-6, v_other: Optional[torch.Tensor] = None, lam: float = 0.0,
+                            q_weight: Optional[torch.Tensor] = None, k_weight: Optional[torch.Tensor] = None) -> torch.Tensor:
     """q [T, heads * dim], k [T, kv_heads * dim], v [T, kv_heads * vdim] (dense rows of one input product): rotates the first
-    ``rot_dims`` numbers of every q and k head at the row's position, optionally brings every q and k head to unit RMS, blends v
+    ``rot_dims`` numbers of every q and k head at the row's position, optionally brings every q and k head to unit RMS (times ``q_weight`` /
+    ``k_weight`` [dim], applied before the rotation), blends v
     with ``v_other`` ((1 - lam) v + lam v_other), writes k and v into the paged caches k_cache [blocks, block, kv_heads, dim] /
     v_cache [.., vdim] at ``slot_mapping`` and returns the prepared queries [T, heads * dim]."""
-    _cuda(q, k, v, k_cache, v_cache, slot_mapping, q_start, ctx_len, seq_of_token, inv_freq, v_other)
+    _cuda(q, k, v, k_cache, v_cache, slot_mapping, q_start, ctx_len, seq_of_token, inv_freq, v_other, q_weight, k_weight)
     nb, bs, G, d = k_cache.shape
     e = v_cache.shape[3]
     T, S = q.shape[0], q_start.numel()
@@ -828,10 +894,36 @@ def rotary_qk_norm_kv_write(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, k
     if v_other is not None:
         _need(v_other.dtype == v.dtype and v_other.shape[0] == T, "rotary_qk_norm_kv_write: v_other [T, kv_heads * vdim]")
         vos = _rows(v_other, G * e, "v_other")
+    _need((q_weight is None) == (k_weight is None) and (q_weight is None or qk_norm), "rotary_qk_norm_kv_write: weights belong to the norm")
+    for w in (q_weight, k_weight):
+        _need(w is None or (w.dtype == q.dtype and w.numel() == d and w.is_contiguous()), "rotary_qk_norm_kv_write: weights [dim]")
     q_out = torch.empty(T, H * d, dtype=q.dtype, device=q.device)
     check(_lib.mixers_lib().aphro_rotary_qk_norm_kv_write(
         q_out.data_ptr(), H * d, k_cache.data_ptr(), v_cache.data_ptr(), slot_mapping.data_ptr(), nb * bs, q.data_ptr(),
         _rows(q, H * d, "q"), k.data_ptr(), _rows(k, G * d, "k"), v.data_ptr(), _rows(v, G * e, "v"), _p(v_other), vos, float(lam),
         q_start.data_ptr(), ctx_len.data_ptr(), seq_of_token.data_ptr(), _p(inv_freq), T, H, G, d, e, int(rot_dims), int(layout),
-        1 if qk_norm else 0, float(eps), _dt(q), _stream()), "rotary_qk_norm_kv_write")
+        1 if qk_norm else 0, _p(q_weight), _p(k_weight), float(eps), _dt(q), _stream()), "rotary_qk_norm_kv_write")
+    return q_out
+
+
+def qk_row_norm_kv_write(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor,
+                         slot_mapping: torch.Tensor, q_weight: torch.Tensor, k_weight: torch.Tensor, eps: float) -> torch.Tensor:
+    """q [T, heads * dim] and k [T, kv_heads * dim] (dense rows) divided by the root mean square of the whole row, times their
+    weights; k and v [T, kv_heads * vdim] go into the paged caches [blocks, block, kv_heads, dim / vdim] at ``slot_mapping``; returns
+    the queries."""
+    _cuda(q, k, v, k_cache, v_cache, slot_mapping, q_weight, k_weight)
+    nb, bs, G, d = k_cache.shape
+    e = v_cache.shape[3]
+    T, nq, nk, nv = q.shape[0], q.shape[1], G * d, G * e
+    _need(v_cache.shape[:3] == (nb, bs, G) and k_cache.is_contiguous() and v_cache.is_contiguous(), "qk_row_norm_kv_write: cache shapes")
+    _need(q.dtype == k.dtype == v.dtype == k_cache.dtype == v_cache.dtype == q_weight.dtype == k_weight.dtype, "qk_row_norm_kv_write: one dtype")
+    _need(k.shape[0] == T and v.shape[0] == T and slot_mapping.dtype == torch.int64 and slot_mapping.numel() == T
+          and slot_mapping.is_contiguous(), "qk_row_norm_kv_write: one row and one slot (int64) per token")
+    _need(q_weight.numel() == nq and k_weight.numel() == nk and q_weight.is_contiguous() and k_weight.is_contiguous(),
+          "qk_row_norm_kv_write: weights as long as the rows")
+    q_out = torch.empty(T, nq, dtype=q.dtype, device=q.device)
+    check(_lib.mixers_lib().aphro_qk_row_norm_kv_write(
+        q_out.data_ptr(), nq, k_cache.data_ptr(), v_cache.data_ptr(), slot_mapping.data_ptr(), nb * bs, q.data_ptr(), _rows(q, nq, "q"),
+        k.data_ptr(), _rows(k, nk, "k"), v.data_ptr(), _rows(v, nv, "v"), q_weight.data_ptr(), k_weight.data_ptr(), T, nq, nk, nv,
+        float(eps), _dt(q), _stream()), "qk_row_norm_kv_write")
     return q_out

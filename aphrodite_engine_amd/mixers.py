@@ -4,7 +4,8 @@ portions and decoded tokens in one launch -- through the kernels of ``mixer_ops`
 
   DistanceBiasAttention   grouped-query softmax attention over a token-major paged cache; no rotation: positions enter as
                           an additive per-head bias looked up by (bucketed) distance and as a query temperature that
-                          grows with the logarithm of the position; optional per-head sigmoid output gate
+                          grows with the logarithm of the position; optional sigmoid output gate (per head or elementwise),
+                          sliding window or chunks, tanh soft cap on the scores, sink in the softmax denominator
   OuterProductMemory      a matrix state per head in a per-request slot: decay linear attention (fixed per-head decay) or
                           the mLSTM cell (exponential gating under a running maximum, normaliser vector)
   LayerNormParams, GatedMLP  the norm with weight and bias around an fp32 residual stream; gate * up feed-forward
@@ -23,8 +24,13 @@ portions and decoded tokens in one launch -- through the kernels of ``mixer_ops`
   ClampedGLUMLP           down(g * sigmoid(alpha g) * (u + 1)) with g and u clamped, biased projections
   StreamedResidual        a residual carried as several streams that sublayers read through a learned combination and write back
                           through a learned mixing matrix (hyper-connections), with a per-channel scale on every sublayer's result
-  GatedDeltaMixer         the gated delta rule: a matrix state per head that forgets, corrects what it holds under the key and is
-                          read after the write; short causal convolutions with silu on q, k and v; unit-norm q and k
+  GatedDeltaMixer         the gated delta rule: a matrix state per head that forgets (as a whole, or every key channel at its own
+                          rate), corrects what it holds under the key and is read after the write; short causal convolutions with
+                          silu on q, k and v; unit-norm q and k; decay and output gate optionally through low-rank products
+  SelectiveStateSpace     Mamba-2: an outer-product memory whose decay and write strength come from a step size per head and token,
+                          keys and queries shared by groups of heads, behind a short convolution; gate, then RMS norm in parts
+  GroupedQueryAttention   softmax attention of a fused input product's q, k and v rows: q / k normed per head before a (partial)
+                          rotation or over the whole projection without one, masks / soft cap / distance bias / sink / gate as above
   RotaryGQAttention       causal grouped-query softmax attention with a (partial) rotation, optional unit RMS of q and k after it
                           and optional blending of the values with an earlier layer's values of the same tokens
 """
@@ -117,8 +123,14 @@ class LayerNormParams(nn.Module):
 
 class DistanceBiasAttention(nn.Module):
     def __init__(self, heads: int, kv_heads: int, dim: int, vdim: int, scale: float, bias_rows: int = 0,
-                 bias_far: float = 0.0, temp_coef: float = 0.0, temp_every: int = 1):
+                 bias_far: float = 0.0, temp_coef: float = 0.0, temp_every: int = 1, window: int = 0, chunk: int = 0,
+                 softcap: float = 0.0, sink: Optional[float] = None):
+        """``window`` > 0: a row sees itself and the window - 1 tokens before it; ``chunk`` > 0: only its own chunk of positions,
+        counted from the sequence's start; ``softcap`` > 0: softcap * tanh(score / softcap) before the bias; ``sink``: a score
+        without key or value that joins every softmax denominator."""
         super().__init__()
+        self.window, self.chunk, self.softcap = max(int(window), 0), max(int(chunk), 0), max(float(softcap), 0.0)
+        self.register_buffer("sink", None if sink is None else torch.full((heads, ), float(sink), dtype=torch.float32), persistent=False)
         if heads % kv_heads:
             raise ValueError(f"{heads} query heads over {kv_heads} key/value heads")
         self.heads, self.kv_heads, self.dim, self.vdim = heads, kv_heads, dim, vdim
@@ -145,10 +157,16 @@ class DistanceBiasAttention(nn.Module):
     def forward(self, out: torch.Tensor, q, k, v, gate, cache, batch: StepBatch, out_scale: float = 1.0) -> None:
         k_cache, v_cache = cache
         mops.paged_kv_write(k_cache, v_cache, k, v, batch.slot_mapping)
+        self.attend(out, q, gate, cache, batch, out_scale)
+
+    def attend(self, out: torch.Tensor, q, gate, cache, batch: StepBatch, out_scale: float = 1.0) -> None:
+        """The attention launch alone, over a cache that already holds the step's own keys and values."""
+        k_cache, v_cache = cache
         mops.distance_bias_attention(out, q, gate, k_cache, v_cache, batch.block_tables, batch.q_start, batch.q_len,
                                      batch.ctx_len, batch.seq_of_token, (min(batch.q_lens), max(batch.q_lens)), self.heads,
                                      self.scale, self.bias_lut, self.temp_coef, self.temp_every, out_scale,
-                                     max_kv_len=max(c + n for c, n in zip(batch.ctx_lens, batch.q_lens)))
+                                     max_kv_len=max(c + n for c, n in zip(batch.ctx_lens, batch.q_lens)), window=self.window,
+                                     chunk=self.chunk, softcap=self.softcap, sink=self.sink)
 
 
 class OuterProductMemory(nn.Module):
@@ -521,10 +539,13 @@ class GatedDeltaMixer(nn.Module):
     time with silu (its last inputs live in a per-request slot); q and k become unit vectors per head (q also times dim^-1/2);
     per head  S <- g S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q  with beta = sigmoid(.), g = exp(-exp(A_log)
     softplus(. + dt_bias)); o is divided by its root mean square over the head, times a weight shared by the heads, times
-    silu(gate); then the output product.  The state S is fp32 in a per-request slot and starts at zero."""
+    act(gate); then the output product.  The state S is fp32 in a per-request slot and starts at zero.
+
+    ``decay_rank`` > 0: one decay per head and key channel (a row of S each), g = exp(-exp(A_log) softplus(W_a2 W_a1 h + dt_bias)) with
+    an inner size of ``decay_rank``; ``gate_rank`` > 0: the output gate is W_g2 W_g1 h.  The inner rows W_a1 and W_g1 join the input product."""
 
     def __init__(self, width: int, heads: int, kv_heads: int, dim: int, vdim: int, taps: int, eps: float, dtype, prefix: str = "",
-                 norm_eps: float = 1e-6):
+                 norm_eps: float = 1e-6, decay_rank: int = 0, gate_rank: int = 0, gate_act: int = mops.GATE_SILU):
         super().__init__()
         from .loader import merged_plan
         from .model import QuantLinear
@@ -533,18 +554,23 @@ class GatedDeltaMixer(nn.Module):
         if taps < 1:
             raise ValueError("a convolution has at least one tap")
         self.heads, self.kv_heads, self.dim, self.vdim, self.taps = heads, kv_heads, dim, vdim, int(taps)
-        self.eps, self.norm_eps = float(eps), float(norm_eps)
-        self.names = ["q", "k", "v", "g", "b", "a"]
-        self.splits = [kv_heads * dim, kv_heads * dim, heads * vdim, heads * vdim, heads, heads]
+        self.eps, self.norm_eps, self.gate_act = float(eps), float(norm_eps), int(gate_act)
+        self.decay_rank, self.gate_rank = int(decay_rank), int(gate_rank)
+        self.names = ["q", "k", "v", "g1" if gate_rank else "g"] + (["a1", "b"] if decay_rank else ["b", "a"])
+        self.splits = [kv_heads * dim, kv_heads * dim, heads * vdim, self.gate_rank or heads * vdim] + \
+            ([self.decay_rank, heads] if decay_rank else [heads, heads])
+        self.at = {n: sum(self.splits[:i]) for i, n in enumerate(self.names)}
         pad = -sum(self.splits) % 8               # rows of the fused product stay 16-byte multiples
         if pad:
             self.splits.append(pad)
         self.channels = sum(self.splits[:3])
         self.in_proj = QuantLinear(width, self.splits, None, dtype, prefix=prefix + "in_proj", plan=merged_plan(self.splits))
         self.in_proj.weight.data.zero_()
+        self.a2 = QuantLinear(decay_rank, [heads * dim], None, dtype, prefix=prefix + "a2") if decay_rank else None
+        self.g2 = QuantLinear(gate_rank, [heads * vdim], None, dtype, prefix=prefix + "g2") if gate_rank else None
         self.conv = nn.Parameter(torch.zeros(self.channels, self.taps, dtype=dtype), requires_grad=False)
         self.a_log = nn.Parameter(torch.zeros(heads, dtype=torch.float32), requires_grad=False)
-        self.dt_bias = nn.Parameter(torch.zeros(heads, dtype=torch.float32), requires_grad=False)
+        self.dt_bias = nn.Parameter(torch.zeros(heads * dim if decay_rank else heads, dtype=torch.float32), requires_grad=False)
         self.out_norm = nn.Parameter(torch.ones(vdim, dtype=dtype), requires_grad=False)
         self.out_proj = QuantLinear(heads * vdim, [width], None, dtype, prefix=prefix + "out_proj")
 
@@ -552,19 +578,106 @@ class GatedDeltaMixer(nn.Module):
         """(convolution state, matrix state)"""
         return ConvStateSpec(self.channels, self.taps), MemoryStateSpec(self.heads, self.dim, self.vdim, mops.MEMORY_DECAY)
 
-    def forward(self, h: torch.Tensor, conv_state: torch.Tensor, state, batch: StepBatch) -> torch.Tensor:
+    def forward(self, h: torch.Tensor, conv_state: torch.Tensor, state, batch: StepBatch, rows: Optional[torch.Tensor] = None) -> torch.Tensor:
+        """``rows``: only these rows of the result are wanted (the states advance over all of them)."""
         H, G, d, e = self.heads, self.kv_heads, self.dim, self.vdim
         proj = self.in_proj(h)
+        part = lambda name, n: proj[:, self.at[name]:self.at[name] + n]
         qkv = mops.short_conv(proj[:, :self.channels], self.conv, conv_state, batch.state_slots, batch.q_start, batch.q_len,
                               batch.ctx_len, batch.seq_of_token, self.channels, act=1)
-        g_at = self.channels
-        b_at = g_at + H * e
-        o = mops.gated_delta_scan(qkv[:, :G * d], qkv[:, G * d:2 * G * d], qkv[:, 2 * G * d:], proj[:, b_at:b_at + H],
-                                  proj[:, b_at + H:b_at + 2 * H], self.a_log, self.dt_bias, state[0], batch.state_slots,
-                                  batch.q_start, batch.q_len, batch.ctx_len, H, G, d ** -0.5, self.norm_eps, max_q_len=max(batch.q_lens))
-        y = torch.empty(h.shape[0], H * e, dtype=h.dtype, device=h.device)
-        mops.gated_head_rms_norm(y, o, self.out_norm, proj[:, g_at:g_at + H * e], H, self.eps, mops.GATE_SILU)
+        a = self.a2(part("a1", self.decay_rank)) if self.decay_rank else part("a", H)
+        o = mops.gated_delta_scan(qkv[:, :G * d], qkv[:, G * d:2 * G * d], qkv[:, 2 * G * d:], part("b", H), a, self.a_log, self.dt_bias,
+                                  state[0], batch.state_slots, batch.q_start, batch.q_len, batch.ctx_len, H, G, d ** -0.5, self.norm_eps,
+                                  max_q_len=max(batch.q_lens))
+        gate = part("g1", self.gate_rank) if self.gate_rank else part("g", H * e)
+        if rows is not None:
+            o, gate = o.index_select(0, rows), gate.index_select(0, rows)
+        if self.gate_rank:
+            gate = self.g2(gate)
+        y = torch.empty(o.shape[0], H * e, dtype=h.dtype, device=h.device)
+        mops.gated_head_rms_norm(y, o, self.out_norm, gate, H, self.eps, self.gate_act)
         return self.out_proj(y)
+
+
+class SelectiveStateSpace(nn.Module):
+    """Mamba-2, the mechanism only: takes the rows of an input product -- z and x (heads x vdim each), B and C (groups x state each)
+    and one raw step size per head -- and leaves the gated, normed head outputs.  [x | B | C] pass a short causal convolution with bias
+    and silu; dt = softplus(. + dt_bias);  S <- exp(-exp(A_log) dt) S + dt B x^T,  y = S^T C + D x  per head (its group's B and C);
+    y silu(z) is normed in ``norm_groups`` equal parts.  The state is fp32 in a per-request slot, like the convolution's last inputs."""
+
+    def __init__(self, heads: int, vdim: int, state: int, groups: int, taps: int, norm_groups: int, eps: float, dtype):
+        super().__init__()
+        if heads % groups:
+            raise ValueError(f"{heads} heads in {groups} groups")
+        if taps < 1:
+            raise ValueError("a convolution has at least one tap")
+        self.heads, self.vdim, self.state, self.groups, self.taps = heads, vdim, state, groups, int(taps)
+        self.inner, self.norm_groups, self.eps = heads * vdim, int(norm_groups), float(eps)
+        if self.inner % self.norm_groups:
+            raise ValueError(f"{self.inner} channels in {norm_groups} norm groups")
+        self.channels = self.inner + 2 * groups * state
+        self.conv = nn.Parameter(torch.zeros(self.channels, self.taps, dtype=dtype), requires_grad=False)
+        self.conv_bias = nn.Parameter(torch.zeros(self.channels, dtype=dtype), requires_grad=False)
+        self.a_log, self.dt_bias, self.skip = (nn.Parameter(torch.zeros(heads, dtype=torch.float32), requires_grad=False) for _ in range(3))
+        self.norm = nn.Parameter(torch.ones(self.inner, dtype=dtype), requires_grad=False)
+
+    def cache_specs(self):
+        """(convolution state, matrix state)"""
+        return ConvStateSpec(self.channels, self.taps), MemoryStateSpec(self.heads, self.state, self.vdim, mops.MEMORY_STATE_SPACE)
+
+    def forward(self, out: torch.Tensor, xbc: torch.Tensor, z: torch.Tensor, dt: torch.Tensor, conv_state: torch.Tensor, state,
+                batch: StepBatch, out_scale: float = 1.0) -> None:
+        n, gn = self.inner, self.groups * self.state
+        xbc = mops.short_conv(xbc, self.conv, conv_state, batch.state_slots, batch.q_start, batch.q_len, batch.ctx_len,
+                              batch.seq_of_token, self.channels, act=1, bias=self.conv_bias)
+        y = mops.outer_memory_scan(xbc[:, n + gn:], xbc[:, n:n + gn], xbc[:, :n], state, batch.state_slots, batch.q_start, batch.q_len,
+                                   batch.ctx_len, self.heads, mops.MEMORY_STATE_SPACE, gate_i=dt, max_q_len=max(batch.q_lens),
+                                   qk_heads=self.groups, a_log=self.a_log, dt_bias=self.dt_bias, skip=self.skip)
+        mops.silu_gate_part_rms_norm(out, y, z, self.norm, self.norm_groups, self.eps, out_scale)
+
+
+class GroupedQueryAttention(nn.Module):
+    """Grouped-query softmax attention over a token-major paged cache, the mechanism only: takes the q, k and v rows of an input
+    product (and the raw rows of an elementwise sigmoid gate) and leaves the heads' outputs.  ``qk_norm``: None, "head" (RMS norm of
+    every head with a weight shared by the heads, before the rotation) or "row" (RMS norm over the whole projection; no rotation).
+    ``rotary`` turns the first ``rotary.dims`` numbers of every head in the given pair ``layout``.  Masks, soft cap, distance bias and
+    sink are DistanceBiasAttention's, whose kernels it runs."""
+
+    def __init__(self, heads: int, kv_heads: int, dim: int, vdim: int, scale: float, eps: float, dtype, qk_norm: Optional[str] = None,
+                 rotary: Optional[RotaryFrequencies] = None, layout: int = mops.ROTARY_HALF, **attention):
+        super().__init__()
+        if qk_norm not in (None, "head", "row"):
+            raise ValueError(f"qk_norm {qk_norm!r}")
+        if qk_norm == "row" and rotary is not None and rotary.dims:
+            raise ValueError("a rotation after a norm over the whole projection is not served")
+        if rotary is not None and rotary.dims > dim:
+            raise ValueError(f"{rotary.dims} rotated numbers in a head of {dim}")
+        self.heads, self.kv_heads, self.dim, self.vdim, self.eps = heads, kv_heads, dim, vdim, float(eps)
+        self.qk_norm, self.layout = qk_norm, int(layout)
+        self.rotary = rotary if rotary is not None else RotaryFrequencies(0, 1.0)
+        self.attn = DistanceBiasAttention(heads, kv_heads, dim, vdim, scale, **attention)
+        self.splits = [heads * dim, kv_heads * dim, kv_heads * vdim]
+        nq, nk = (heads * dim, kv_heads * dim) if qk_norm == "row" else (dim, dim)
+        self.q_norm = nn.Parameter(torch.ones(nq, dtype=dtype), requires_grad=False) if qk_norm else None
+        self.k_norm = nn.Parameter(torch.ones(nk, dtype=dtype), requires_grad=False) if qk_norm else None
+
+    def cache_spec(self) -> PagedKVSpec:
+        return self.attn.cache_spec()
+
+    def finalize(self, device) -> None:
+        self.rotary.to(device)
+        self.attn.finalize()
+
+    def forward(self, out: torch.Tensor, q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, gate: Optional[torch.Tensor], cache,
+                batch: StepBatch, out_scale: float = 1.0) -> None:
+        k_cache, v_cache = cache
+        if self.qk_norm == "row":
+            q = mops.qk_row_norm_kv_write(q, k, v, k_cache, v_cache, batch.slot_mapping, self.q_norm, self.k_norm, self.eps)
+        else:
+            q = mops.rotary_qk_norm_kv_write(q, k, v, k_cache, v_cache, batch.slot_mapping, batch.q_start, batch.ctx_len,
+                                             batch.seq_of_token, self.rotary.inv_freq, self.rotary.dims, self.layout,
+                                             self.qk_norm is not None, self.eps, q_weight=self.q_norm, k_weight=self.k_norm)
+        self.attn.attend(out, q, gate, cache, batch, out_scale)
 
 
 class RotaryGQAttention(nn.Module):

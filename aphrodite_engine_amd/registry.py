@@ -64,9 +64,14 @@ def _register_builtin() -> None:
         from .pagulix import load_pagulix
         return load_pagulix(model_dir, config, **kw)
 
+    def nukezen(model_dir, config, **kw):
+        from .nukezen import load_nukezen
+        return load_nukezen(model_dir, config, **kw)
+
     for arch in ("LlamaForCausalLM", "MistralForCausalLM", "MixtralForCausalLM"):
         _LOADERS.setdefault(arch, llama)
     _LOADERS.setdefault("Fatudra", fatudra)
     _LOADERS.setdefault("Gipozen", gipozen)
     _LOADERS.setdefault("Fekotar", fekotar)
     _LOADERS.setdefault("Pagulix", pagulix)
+    _LOADERS.setdefault("Nukezen", nukezen)

@@ -30,9 +30,10 @@ extern "C" {
 
 const char* aphro_mixers_last_error(void);
 
-/* residual[t, :] = table[ids[t], :] * scale   (fp32 residual [T, width]; table [vocab, width] of `dtype`) */
+/* residual[t, :] = table[ids[t], :] * scale   (fp32 residual [T, width]; table [vocab, width] of `dtype`); copy [T, width] of
+ * `dtype` takes the same rows rounded (NULL: none) */
 int aphro_embed_scale_f32(float* residual, const void* table, const int64_t* ids, int64_t num_tokens, int width,
-                          int64_t vocab, float scale, int dtype, void* stream);
+                          int64_t vocab, float scale, void* copy, int dtype, void* stream);
 
 /* One launch around an fp32 residual stream r [T, width], every step optional (NULL pointers switch it off):
  *   1. r += layer_norm(y + y_bias; post_w, post_b)      y [T, width] of `dtype` (row stride y_stride), y_bias fp32 [width]
@@ -42,6 +43,20 @@ int aphro_embed_scale_f32(float* residual, const void* table, const int64_t* ids
 int aphro_residual_layer_norm(float* residual, const void* y, int64_t y_stride, const float* y_bias, const void* post_w,
                               const void* post_b, const void* add_vec, const void* pre_w, const void* pre_b, void* out,
                               int64_t num_tokens, int width, float eps, int dtype, void* stream);
+
+/* A sublayer's result joins the residual through a norm of its own, and the next sublayer reads the residual:
+ *   r += y / sqrt(mean(y^2) + eps) * post_w        (y NULL: not)
+ *   out = r / sqrt(mean(r^2) + eps) * pre_w        (pre_w NULL: out = r rounded to `dtype`; out NULL: not written)
+ * r fp32 [T, width], y [T, width] (row stride), post_w, pre_w [width], out [T, width] of `dtype`. */
+int aphro_residual_post_rms_norm(float* residual, const void* y, int64_t y_stride, const void* post_w, const void* pre_w,
+                                 void* out, int64_t num_tokens, int width, float eps, int dtype, void* stream);
+
+/* out[t, i] = out_scale * z[t, i] / sqrt(mean over the part of z^2 + eps) * weight[i],  z = x * silu(gate)   (the gate first):
+ * a row's n numbers form n / part equal parts of neighbours with a root mean square each.  x fp32 [T, n] contiguous; gate and out
+ * [T, n] (row strides), weight [n] of `dtype`. */
+int aphro_silu_gate_part_rms_norm(void* out, int64_t out_stride, const float* x, const void* gate, int64_t gate_stride,
+                                  const void* weight, int64_t num_tokens, int n, int part, float eps, float out_scale, int dtype,
+                                  void* stream);
 
 /* out[t, j] = act(in[t, j]) * in[t, d + j], j < d.  act: 0 silu, 1 gelu (tanh form).  in [T, 2 d] (row stride in_stride),
  * out [T, d] contiguous; math in fp32, one rounding. */
@@ -62,15 +77,19 @@ int aphro_paged_kv_write(void* k_cache, void* v_cache, const void* k, int64_t k_
                          int dtype, void* stream);
 
 /* Causal softmax attention of a batch of segments over the paged cache (which already holds the segments' own keys):
- *   score(i, j) = temp(i) * scale * q_i . k_j + bias_lut[h, min(i - j, lut_len - 1)]
+ *   score(i, j) = cap(temp(i) * scale * q_i . k_j) + bias_lut[h, min(i - j, lut_len - 1)]
+ *   cap(s) = softcap * tanh(s / softcap)                                  (softcap 0: cap(s) = s)
  *   temp(i) = 1 + temp_coef * ln(floor((i + 1) / temp_every) + 1)         (temp_coef == 0: none)
- *   out[t, h, :] = out_scale * sigmoid(gate[t, h]) * sum_j softmax_j(score) v_j     (gate NULL: no gate)
- * q [T, heads * dim] (row stride), gate [T, heads] (row stride) and out [T, heads * vdim] (row stride) of `dtype`;
+ *   row i sees key j if j <= i, i - j < window (window 0: any) and floor(i / chunk) == floor(j / chunk) (chunk 0: any)
+ *   p(i, j) = exp(score) / (exp(sink[h]) + sum_j exp(score))              (sink fp32 [heads]; NULL: the plain softmax)
+ *   out[t, h, :] = out_scale * sigmoid(gate) * sum_j p(i, j) v_j          (gate NULL: no gate; [T, heads], or
+ *                                                                          gate_cols 1: elementwise [T, heads * vdim])
+ * q [T, heads * dim] (row stride), gate (row stride) and out [T, heads * vdim] (row stride) of `dtype`;
  * bias_lut fp32 [heads, lut_len] (NULL: no bias); block_tables int32 [num_seqs, max_blocks]; seq_of_token int32 [T].
  * Query head h reads key/value head h / (heads / kv_heads).  q_len int32 [num_seqs] with its host-side minimum and
  * maximum choose the kernels: bf16 segments of 8 rows or more run on the matrix cores (dim, vdim in {32, 64, 96, 128}),
  * shorter ones on a kernel that reads each key once for all query heads of its kv head (dim, vdim multiples of 8, at most
- * 256, 1 / 2 / 4 / 8 query heads per kv head); every other case -- and fp32 -- runs the scalar fp32 kernel.
+ * 256; up to 8 query heads of a kv head per workgroup); every other case -- and fp32 -- runs the scalar fp32 kernel.
  * max_kv_len (host-side longest ctx_len + q_len) and an optional fp32 workspace let the shared-key kernel split long key
  * ranges over up to 8 workgroups per row (num_tokens * heads * splits * (2 + vdim) floats; NULL: no split). */
 int aphro_distance_bias_attention(void* out, int64_t out_stride, const void* q, int64_t q_stride, const void* gate,
@@ -79,14 +98,18 @@ int aphro_distance_bias_attention(void* out, int64_t out_stride, const void* q, 
                                   const int32_t* q_len, const int32_t* ctx_len, const int32_t* seq_of_token,
                                   int64_t num_tokens, int num_seqs, int min_q_len, int max_q_len, int heads, int kv_heads,
                                   int dim, int vdim, float scale, const float* bias_lut, int lut_len, float temp_coef,
-                                  int temp_every, float out_scale, int max_kv_len, float* workspace,
-                                  int64_t workspace_floats, int dtype, void* stream);
+                                  int temp_every, float out_scale, int window, int chunk, float softcap, const float* sink,
+                                  int gate_cols, int max_kv_len, float* workspace, int64_t workspace_floats, int dtype,
+                                  void* stream);
 
 /* Gated outer-product memory, one state per (slot, head):  S <- a_t S + b_t k_t v_t^T,  o_t = S^T q_t  [/ normaliser].
  *   mode 0 (decay linear attention): q, k, v = silu(raw); a_t = decay[h], b_t = 1.
  *   mode 1 (mLSTM): q = raw * q_scale; log gates i = cap tanh(raw_i / cap), f = logsigmoid(cap tanh(raw_f / cap));
  *     m_t = max(f + m_(t-1), i), a_t = exp(f + m_(t-1) - m_t), b_t = exp(i - m_t); n <- a_t n + b_t k_t;
  *     o_t = S^T q_t / (max(|n . q_t|, exp(-m_t)) + 1e-6).  m, n and S start at zero.
+ *   mode 2 (selective state space): dt = softplus(gate_i + dt_bias[h]), a_t = exp(-exp(a_log[h]) dt), b_t = dt,
+ *     o_t = S^T q_t + skip[h] v_t; q, k [T, qk_heads * dim], head h uses number h / (heads / qk_heads) (modes 0, 1: qk_heads ==
+ *     heads); a_log, dt_bias, skip fp32 [heads].
  * q, k [T, heads * dim], v [T, heads * vdim], gates [T, heads] (row strides) of `dtype`; out fp32 [T, heads * vdim].
  * state_s fp32 [slots, heads, dim, vdim]; mode 1 only: state_n fp32 [slots, heads, tiles, dim] and state_m fp32
  * [slots, heads, tiles], tiles = ceil(vdim / 16) (every 16 value columns keep their own copy of n and m, so no workgroup
@@ -98,7 +121,7 @@ int aphro_outer_memory_scan(float* out, const void* q, int64_t q_stride, const v
                             float* state_n, float* state_m, const int32_t* slot_of_seq, int num_slots,
                             const int32_t* q_start, const int32_t* q_len, const int32_t* ctx_len, int num_seqs,
                             int64_t num_tokens, int heads, int dim, int vdim, int mode, const float* decay, float q_scale,
-                            float gate_cap, int max_q_len, int dtype, void* stream);
+                            float gate_cap, int qk_heads, const float* a_log, const float* dt_bias, const float* skip, int max_q_len, int dtype, void* stream);
 
 /* ---- an fp32 residual stream joined over depth, scalar-gain RMS norm ---------------------------------------------------
  * One launch, every step optional:
@@ -124,14 +147,15 @@ int aphro_differential_norm_gate(void* out, int64_t out_stride, const float* a, 
                                  float out_scale, float eps, int dtype, void* stream);
 
 /* Short causal convolution over time on each channel of u [T, cq + ck + cv] (row stride u_stride):
- *   y_t[c] = sum_j w[c, j] * u_(t - taps + 1 + j)[c],  zeros before the sequence's start;  w [channels, taps] of `dtype`.
+ *   y_t[c] = sum_j w[c, j] * u_(t - taps + 1 + j)[c] + bias[c],  zeros before the sequence's start;  w [channels, taps] and
+ * bias [channels] of `dtype` (bias NULL: none).
  * Channels [0, cq) go to q_out [T, cq] (row stride); [cq, cq + ck) and the last cv go into the token-major paged caches
  * k_cache [cache slots, ck] / v_cache [cache slots, cv] at row cache_slots[t] (int64; outside 0 .. num_cache_slots - 1: skipped).
  * ck == cv == 0: no cache.  state [state slots, taps - 1, channels] of `dtype` holds each request's last taps - 1 inputs:
  * read for the rows before a segment (never for positions before the sequence's start), rewritten afterwards.
  * 1 <= taps <= 16.  act: 0 none, 1 silu on the convolution's result. */
 int aphro_short_conv(void* q_out, int64_t q_out_stride, void* k_cache, void* v_cache, const int64_t* cache_slots,
-                     int64_t num_cache_slots, const void* u, int64_t u_stride, const void* w, void* state,
+                     int64_t num_cache_slots, const void* u, int64_t u_stride, const void* w, const void* bias, void* state,
                      const int32_t* state_slots, const int32_t* q_start, const int32_t* q_len, const int32_t* ctx_len,
                      const int32_t* seq_of_token, int64_t num_tokens, int num_seqs, int cq, int ck, int cv, int taps, int act,
                      int dtype, void* stream);
@@ -283,14 +307,15 @@ int aphro_logit_softcap(float* out, const void* in, int64_t n, float scale, floa
  *   S <- g S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q      (the read-out sees the current token's write)
  * q, k [T, kv_heads * dim] are made unit vectors per head here (x / sqrt(sum x^2 + norm_eps); q times q_scale); value head h
  * uses query / key head h / (heads / kv_heads); v [T, heads * vdim]; beta = sigmoid(b), g = exp(-exp(a_log[h]) *
- * softplus(a + dt_bias[h])) from b, a [T, heads] (row strides, `dtype`); a_log, dt_bias fp32 [heads].  out fp32 [T, heads * vdim].
+ * softplus(a + dt_bias[h])) from b, a [T, heads] (row strides, `dtype`); a_log, dt_bias fp32 [heads].  channel_decay 1: one decay per
+ * head and key channel (row of S), a [T, heads * dim], dt_bias fp32 [heads * dim], a_log per head.  out fp32 [T, heads * vdim].
  * state fp32 [slots, heads, dim, vdim]; a segment with ctx_len == 0 starts from zero without reading its slot.  dim <= 256.
  * max_q_len (host: longest segment) picks the work split. */
 int aphro_gated_delta_scan(float* out, const void* q, int64_t q_stride, const void* k, int64_t k_stride, const void* v,
                            int64_t v_stride, const void* b, int64_t b_stride, const void* a, int64_t a_stride, const float* a_log,
                            const float* dt_bias, float* state, const int32_t* slot_of_seq, int num_slots, const int32_t* q_start,
                            const int32_t* q_len, const int32_t* ctx_len, int num_seqs, int64_t num_tokens, int heads, int kv_heads,
-                           int dim, int vdim, float q_scale, float norm_eps, int max_q_len, int dtype, void* stream);
+                           int dim, int vdim, int channel_decay, float q_scale, float norm_eps, int max_q_len, int dtype, void* stream);
 /* out[t, h, i] = x[t, h, i] / sqrt(mean_i x^2 + eps) * weight[i] * act(gate[t, h, i]); x fp32 [T, heads * vdim] contiguous;
  * weight [vdim] (shared by the heads; NULL: ones), gate (row stride; NULL: none) and out (row stride) of `dtype`;
  * act 0: sigmoid, 1: silu. */
@@ -300,7 +325,8 @@ int aphro_gated_head_rms_norm(void* out, int64_t out_stride, const float* x, con
 
 /* From the rows of a rotary attention's input product: the first rot_dims numbers of every query and key head turned by
  * position * inv_freq[i] (layout 0: number i pairs with i + rot_dims / 2; 1: number 2 i with 2 i + 1), then -- qk_norm != 0 --
- * every query and key head divided by sqrt(mean(x^2) + eps); values blended v <- (1 - lambda) v + lambda v_other (v_other NULL:
+ * every query and key head divided by sqrt(mean(x^2) + eps), times -- before the rotation -- q_weight [dim] or k_weight [dim] of
+ * `dtype`, shared by the heads (NULL: none); values blended v <- (1 - lambda) v + lambda v_other (v_other NULL:
  * none).  Queries go to q_out [T, heads * dim], keys and values into k_cache [rows, kv_heads, dim] / v_cache [rows, kv_heads,
  * vdim] at slot_mapping[t] (outside 0 .. num_cache_rows - 1: skipped).  dim <= 512. */
 int aphro_rotary_qk_norm_kv_write(void* q_out, int64_t q_out_stride, void* k_cache, void* v_cache, const int64_t* slot_mapping,
@@ -308,7 +334,15 @@ int aphro_rotary_qk_norm_kv_write(void* q_out, int64_t q_out_stride, void* k_cac
                                   const void* v, int64_t v_stride, const void* v_other, int64_t v_other_stride, float lambda,
                                   const int32_t* q_start, const int32_t* ctx_len, const int32_t* seq_of_token, const float* inv_freq,
                                   int64_t num_tokens, int heads, int kv_heads, int dim, int vdim, int rot_dims, int layout,
-                                  int qk_norm, float eps, int dtype, void* stream);
+                                  int qk_norm, const void* q_weight, const void* k_weight, float eps, int dtype, void* stream);
+
+/* An attention's preparation without rotation: q [T, nq] and k [T, nk] (row strides), every row at once divided by
+ * sqrt(mean(row^2) + eps) and times q_weight [nq] / k_weight [nk]; queries go to q_out [T, nq], keys and the values v [T, nv] as
+ * they are into k_cache [rows, nk] / v_cache [rows, nv] at slot_mapping[t] (outside 0 .. num_cache_rows - 1: skipped). */
+int aphro_qk_row_norm_kv_write(void* q_out, int64_t q_out_stride, void* k_cache, void* v_cache, const int64_t* slot_mapping,
+                               int64_t num_cache_rows, const void* q, int64_t q_stride, const void* k, int64_t k_stride,
+                               const void* v, int64_t v_stride, const void* q_weight, const void* k_weight, int64_t num_tokens,
+                               int nq, int nk, int nv, float eps, int dtype, void* stream);
 
 #ifdef __cplusplus
 }

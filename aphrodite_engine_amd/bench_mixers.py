@@ -1,4 +1,4 @@
-"""``bench.py --mixers [--mixers-design fatudra|gipozen|fekotar|pagulix]``: prefill and decode throughput of a Fatudra (or Gipozen) stack at sizes that resemble a real model's layers
+"""``bench.py --mixers [--mixers-design fatudra|gipozen|fekotar|pagulix|nukezen]``: prefill and decode throughput of a Fatudra (or Gipozen) stack at sizes that resemble a real model's layers
 (random bf16 weights), beside a Llama stack of equal width / heads / feed-forward / layer count on the unquantised op path,
 plus each mixer kernel alone against its roofline and against the like kernel of the Llama path.  Prints ONE JSON line;
 the default workload of bench.py is untouched by it.  The Gipozen stack: windowed differential attention (two maps of half the
@@ -15,6 +15,12 @@ The Pagulix stack: a gated-delta layer (16 / 32 value heads of 128 x 128 state o
 latent attention layer (rank 512 + 64 rotated numbers, window 1024, sinks), two rotary attention layers with unit-RMS q / k and
 blended values, four residual streams, 16 silu experts (top 4, softmax over the chosen) plus a shared expert in every layer; it
 stands beside the Fekotar stack (the closest existing model) and Llama.
+
+The Nukezen stack: a channel-delta layer (16 / 32 heads of 128 x 128 state, inner sizes of 128, 4-tap convolutions), two layers of a
+1024-token window attention beside a selective state space (twice the width, heads of 64, state 128, 8 groups) that share their
+tensors, and a chunked attention layer (chunks of 2048, soft cap, distance bias, sink), a dense gelu feed-forward in every layer; it
+stands beside the Fatudra stack (the closest existing model: attention beside a memory, post-norms, the same feed-forward), the
+Pagulix stack (the other delta rule) and Llama.
 
 Rooflines used: 8 TB/s HBM for the memory-bound kernels (norms, activations, decode attention, the decode step of the
 memories: their state is read and written once), 2.5 PFLOP/s dense bf16 MFMA for prompt attention (4 d flops per visible
@@ -649,10 +655,178 @@ def main_pagulix(args) -> int:
     return 0
 
 
+NUK_WINDOW, NUK_CHUNK, NUK_TAPS, NUK_RANK, NUK_STATE, NUK_SSM_VDIM, NUK_GROUPS, NUK_REL, NUK_FAR = 1024, 2048, 4, 128, 128, 64, 8, 32, 2048
+
+
+def nukezen_config(s):
+    """channel delta, window attention beside a state space (twice, on one layer's tensors), chunked attention; dense feed-forwards.
+    Returns (config, shapes of the tensors whose sizes a config leaves open)."""
+    H, G, d = s["heads"], s["kv_heads"], s["dim"]
+    dense = {"kind": "dense", "ff": s["ff"]}
+    delta = {"type": "channel_delta", "mixer": {"heads": H, "kv_heads": H, "dim": d, "vdim": d, "conv": NUK_TAPS}, "mlp": dense}
+    par = {"type": "parallel", "mlp": dense,
+           "mixer": {"left": {"heads": H, "kv_heads": G, "dim": d, "vdim": d, "mask": {"size": NUK_WINDOW},
+                              "rot": {"base": 500000.0, "dims": d}, "scale": d ** -0.5},
+                     "right": {"heads": 2 * s["width"] // NUK_SSM_VDIM, "vdim": NUK_SSM_VDIM, "state": NUK_STATE, "groups": NUK_GROUPS,
+                               "norm_groups": NUK_GROUPS, "conv": NUK_TAPS}, "left_scale": 1.0, "right_scale": 1.0}}
+    attn = {"type": "attention", "mlp": dense,
+            "mixer": {"heads": H, "kv_heads": G, "dim": d, "vdim": d, "mask": {"size": NUK_CHUNK}, "softcap": 30.0, "bias_max": NUK_FAR,
+                      "scale": d ** -0.5}}
+    layers = [delta, par, attn, dict(par, weights_of=1)][:LAYERS]
+    return {"architecture": "Nukezen", "vocab": VOCAB, "width": s["width"], "norm": {"eps": 1e-6}, "embedding": {"scale": 1.0},
+            "layers": layers}, {"l0.mix.a1": (NUK_RANK, s["width"]), "l0.mix.g1": (NUK_RANK, s["width"]), "l2.mix.rel": (NUK_REL, H)}
+
+
+def nukezen_kernel_section(s, prompt_len, batch, ctx, device):
+    """Each kernel that Nukezen adds (or extends) alone at the stack's shapes, beside the like kernel of the closest existing path."""
+    from . import mixer_ops as mops
+    from .mixers import DistanceBiasAttention, RotaryFrequencies
+    bf = torch.bfloat16
+    H, G, d, W = s["heads"], s["kv_heads"], s["dim"], s["width"]
+    SH, SE, N, SG = 2 * W // NUK_SSM_VDIM, NUK_SSM_VDIM, NUK_STATE, NUK_GROUPS
+    pre, dec, pages = batches(prompt_len, batch, ctx, device, VOCAB)
+    out = {}
+
+    def rec(name, sec, like, lsec, bytes_=None, flops=None, lbytes=None, lflops=None):
+        """lbytes / lflops: the like kernel's work where it differs."""
+        r, lr = {"us": round(sec * 1e6, 1)}, {"kernel": like, "us": round(lsec * 1e6, 1)}
+        if bytes_ is not None:
+            r["frac_hbm"], lr["frac_hbm"] = round(bytes_ / sec / HBM, 3), round((lbytes or bytes_) / lsec / HBM, 3)
+        if flops is not None:
+            r["frac_mfma"], lr["frac_mfma"] = round(flops / sec / MFMA, 5), round((lflops or flops) / lsec / MFMA, 5)
+        r["like"] = lr
+        out[name] = r
+
+    rn = lambda *shape, dtype=bf: torch.randn(*shape, device=device, dtype=dtype)
+    rot = RotaryFrequencies(d, 500000.0).to(device)
+    kc, vc = rn(pages, BLOCK, G, d), rn(pages, BLOCK, G, d)
+    att = DistanceBiasAttention(H, G, d, d, d ** -0.5, bias_rows=NUK_REL, bias_far=float(NUK_FAR)).to(device)
+    att.rel.normal_()
+    att.finalize()
+    sink = torch.zeros(H, device=device)
+    for name, b, T in (("prefill", pre, prompt_len), ("decode", dec, batch)):
+        seg = (b.state_slots, b.q_start, b.q_len, b.ctx_len)
+        lens = (min(b.q_lens), max(b.q_lens))
+        kvmax = max(c + q for c, q in zip(b.ctx_lens, b.q_lens))
+        # ---- the residual's launch, the embedding's ---------------------------------------------------------------------------
+        x, y, w16 = rn(T, W, dtype=torch.float32), rn(T, W), rn(W)
+        sec = timed(lambda: mops.residual_post_rms_norm(x, y, w16))
+        lsec = timed(lambda: mops.residual_layer_norm(x, y=y, post=(w16, w16), pre=(w16, w16)))
+        rec("residual_post_rms_norm_" + name, sec, "residual_layer_norm", lsec, bytes_=T * W * 12)
+        # ---- preparation of the two attentions ------------------------------------------------------------------------------------
+        q, k, v, g = rn(T, H * d), rn(T, G * d), rn(T, G * d), rn(T, H * d)
+        wh, wq, wk = rn(d), rn(H * d), rn(G * d)
+        pb = T * (2 * H + 4 * G) * d * 2
+        prep = lambda layout, **kw: mops.rotary_qk_norm_kv_write(q, k, v, kc, vc, b.slot_mapping, b.q_start, b.ctx_len, b.seq_of_token,
+                                                                 rot.inv_freq, d, layout, True, 1e-6, **kw)
+        sec = timed(lambda: prep(mops.ROTARY_INTERLEAVED, q_weight=wh, k_weight=wh))
+        lsec = timed(lambda: prep(mops.ROTARY_HALF))
+        rec("rotary_qk_norm_kv_write_" + name, sec, "rotary_qk_norm_kv_write without weights", lsec, bytes_=pb)
+        sec = timed(lambda: mops.qk_row_norm_kv_write(q, k, v, kc, vc, b.slot_mapping, wq, wk, 1e-6))
+        rec("qk_row_norm_kv_write_" + name, sec, "rotary_qk_norm_kv_write without weights", lsec, bytes_=pb)
+        # ---- the attentions -----------------------------------------------------------------------------------------------------------
+        o = torch.empty(T, H * d, device=device, dtype=bf)
+        run = lambda gate=None, lut=None, **kw: mops.distance_bias_attention(
+            o, q, gate, kc, vc, b.block_tables, b.q_start, b.q_len, b.ctx_len, b.seq_of_token, lens, H, d ** -0.5, lut, max_kv_len=kvmax, **kw)
+        wsec = timed(lambda: run(gate=g, window=NUK_WINDOW))
+        csec = timed(lambda: run(lut=att.bias_lut, chunk=NUK_CHUNK, softcap=30.0, sink=sink))
+        lsec, lbsec = timed(lambda: run()), timed(lambda: run(lut=att.bias_lut))
+        if name == "prefill":
+            per = H * 4.0 * d
+            pairs = T * (T + 1) / 2
+            wp, cp = sum(min(i + 1, NUK_WINDOW) for i in range(T)), sum(i % NUK_CHUNK + 1 for i in range(T))
+            rec("window_attention_prefill", wsec, "the same launch, causal, no gate", lsec, flops=wp * per, lflops=pairs * per)
+            rec("chunked_attention_prefill", csec, "the same launch, causal, distance bias alone", lbsec, flops=cp * per, lflops=pairs * per)
+        else:
+            per = batch * G * 2 * d * 2
+            rec("window_attention_decode", wsec, "the same launch, causal, no gate", lsec, bytes_=min(ctx + 1, NUK_WINDOW) * per, lbytes=(ctx + 1) * per)
+            rec("chunked_attention_decode", csec, "the same launch, causal, distance bias alone", lbsec, bytes_=(ctx % NUK_CHUNK + 1) * per,
+                lbytes=(ctx + 1) * per)
+        # ---- the delta rule, one decay per channel ---------------------------------------------------------------------------------
+        dk, dv, bb, ca, ha = rn(T, H * d), rn(T, H * d), rn(T, H), rn(T, H * d), rn(T, H)
+        a_log, dtc, dth = torch.zeros(H, device=device), torch.zeros(H * d, device=device), torch.zeros(H, device=device)
+        state = torch.zeros(batch, H, d, d, device=device)
+        scan = lambda a, dt: mops.gated_delta_scan(q, dk, dv, bb, a, a_log, dt, state, *seg, H, H, d ** -0.5, 1e-6, max_q_len=lens[1])
+        sec, lsec = timed(lambda: scan(ca, dtc)), timed(lambda: scan(ha, dth))
+        if name == "prefill":
+            rec("channel_delta_scan_prefill", sec, "gated_delta_scan", lsec, flops=T * H * 4.0 * d * d)
+        else:
+            rec("channel_delta_scan_decode", sec, "gated_delta_scan", lsec, bytes_=batch * H * d * d * 8)
+        o32, yo = rn(T, H * d, dtype=torch.float32), torch.empty(T, H * d, device=device, dtype=bf)
+        sec = timed(lambda: mops.gated_head_rms_norm(yo, o32, wh, g, H, 1e-6, mops.GATE_SIGMOID))
+        lsec = timed(lambda: mops.gated_head_rms_norm(yo, o32, wh, g, H, 1e-6, mops.GATE_SILU))
+        rec("gated_head_rms_norm_sigmoid_" + name, sec, "gated_head_rms_norm with silu", lsec, bytes_=T * H * d * 8)
+        # ---- the state space ------------------------------------------------------------------------------------------------------------
+        C = SH * SE + 2 * SG * N
+        u, cw, cb = rn(T, C), rn(C, NUK_TAPS), rn(C)
+        cst = torch.zeros(batch, NUK_TAPS - 1, C, device=device, dtype=bf)
+        conv = lambda **kw: mops.short_conv(u, cw, cst, *seg, b.seq_of_token, C, act=1, **kw)
+        sec, lsec = timed(lambda: conv(bias=cb)), timed(lambda: conv())
+        rec("short_conv_bias_" + name, sec, "short_conv without bias", lsec, bytes_=T * C * 4)
+        xv, Bm, Cm, dt = u[:, :SH * SE], u[:, SH * SE:SH * SE + SG * N], u[:, SH * SE + SG * N:], rn(T, SH)
+        sst = torch.zeros(batch, SH, N, SE, device=device)
+        al, db, sk, decay = torch.zeros(SH, device=device), torch.zeros(SH, device=device), torch.ones(SH, device=device), torch.full((SH, ), 0.97, device=device)
+        sec = timed(lambda: mops.outer_memory_scan(Cm, Bm, xv, (sst, ), *seg, SH, mops.MEMORY_STATE_SPACE, gate_i=dt, max_q_len=lens[1],
+                                                   qk_heads=SG, a_log=al, dt_bias=db, skip=sk))
+        qh = rn(T, SH * N)
+        lsec = timed(lambda: mops.outer_memory_scan(qh, qh, xv, (sst, ), *seg, SH, mops.MEMORY_DECAY, decay, max_q_len=lens[1]))
+        if name == "prefill":
+            rec("state_space_scan_prefill", sec, "outer_memory_scan (decay)", lsec, flops=T * SH * 4.0 * N * SE)
+        else:
+            rec("state_space_scan_decode", sec, "outer_memory_scan (decay)", lsec, bytes_=batch * SH * N * SE * 8)
+        y32, z, wn = rn(T, SH * SE, dtype=torch.float32), rn(T, SH * SE), rn(SH * SE)
+        ys = torch.empty(T, SH * SE, device=device, dtype=bf)
+        sec = timed(lambda: mops.silu_gate_part_rms_norm(ys, y32, z, wn, SG, 1e-6))
+        lsec = timed(lambda: mops.gated_group_rms_norm(ys, y32, wn, z, SH * SE // SG, 1e-6))
+        rec("silu_gate_part_rms_norm_" + name, sec, "gated_group_rms_norm", lsec, bytes_=T * SH * SE * 8)
+    return out
+
+
+def main_nukezen(args) -> int:
+    from . import _lib
+    from .fatudra import FatudraConfig, FatudraForCausalLM
+    from .model import LlamaConfig, LlamaForCausalLM
+    from .nukezen import NukezenConfig, NukezenForCausalLM
+    from .pagulix import PagulixConfig, PagulixForCausalLM
+    _lib.lib()
+    _lib.mixers_lib()
+    device = torch.device("cuda", 0)
+    torch.cuda.set_device(device)
+    prompt_len, batch, ctx = args.mixers_prompt, args.batch, args.ctx
+    result = {"metric": "nukezen_vs_llama_bf16_throughput", "unit": "tokens/s", "dtype": "bf16", "data": "synthetic",
+              "n_gpus": 1, "layers": LAYERS, "sizes": {}}
+
+    def llama(s):
+        lc = LlamaConfig(hidden_size=s["width"], intermediate_size=s["ff"], num_hidden_layers=LAYERS,
+                         num_attention_heads=s["heads"], num_key_value_heads=s["kv_heads"], vocab_size=VOCAB,
+                         max_position_embeddings=max(8192, prompt_len + 16))
+        m = LlamaForCausalLM(lc, None, torch.bfloat16).init_synthetic(device)
+        m.use_fused_decode = False
+        return m
+    makers = {"nukezen": lambda s: NukezenForCausalLM(NukezenConfig.from_dict(*nukezen_config(s)), torch.bfloat16).init_synthetic(device),
+              "fatudra": lambda s: FatudraForCausalLM(FatudraConfig.from_dict(fatudra_config(s)), torch.bfloat16).init_synthetic(device),
+              "pagulix": lambda s: PagulixForCausalLM(PagulixConfig.from_dict(pagulix_config(s)), torch.bfloat16).init_synthetic(device),
+              "llama": llama}
+    with torch.no_grad():
+        for name, s in SIZES.items():
+            if args.mixers_size and name != args.mixers_size:
+                continue
+            t0 = time.time()
+            r = {who: model_throughput(make(s), prompt_len, batch, ctx, device, VOCAB) for who, make in makers.items()}
+            r["kernels"] = nukezen_kernel_section(s, prompt_len, batch, ctx, device)
+            r["seconds"] = round(time.time() - t0, 1)
+            result["sizes"][name] = r
+            torch.cuda.empty_cache()
+    print(json.dumps(result), flush=True)
+    return 0
+
+
 def main(args) -> int:
     from . import _lib
     if getattr(args, "mixers_design", "fatudra") == "pagulix":
         return main_pagulix(args)
+    if getattr(args, "mixers_design", "fatudra") == "nukezen":
+        return main_nukezen(args)
     if getattr(args, "mixers_design", "fatudra") == "gipozen":
         return main_gipozen(args)
     if getattr(args, "mixers_design", "fatudra") == "fekotar":

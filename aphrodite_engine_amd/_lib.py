@@ -170,7 +170,7 @@ MIXERS_SIGNATURES = {
     "aphro_mixers_last_error": (ctypes.c_char_p, []),
     "aphro_embed_scale_f32": (I, [P, P, P, L, I, L, F, P, I, P]),
     "aphro_residual_layer_norm": (I, [P, P, L, P, P, P, P, P, P, P, L, I, F, I, P]),
-    "aphro_act_and_mul": (I, [P, P, L, L, I, I, I, P]),
+    "aphro_act_and_mul": (I, [P, L, P, L, L, I, I, I, P]),
     "aphro_gated_group_rms_norm": (I, [P, L, P, P, P, L, L, I, I, F, F, I, P]),
     "aphro_paged_kv_write": (I, [P, P, P, L, P, L, P, L, I, I, I, L, I, P]),
     "aphro_distance_bias_attention": (I, [P, L, P, L, P, L, P, P, P, I, L, I, P, P, P, P, L, I, I, I, I, I, I, I, F, P, I, F,
@@ -199,10 +199,10 @@ MIXERS_SIGNATURES = {
     "aphro_token_state_write": (I, [P, P, P, P, P, I, P]),
     "aphro_residual_add2_rms_norm": (I, [P, P, L, P, L, P, P, P, L, I, F, I, P]),
     "aphro_latent_prep": (I, [P, P, L, P, L, I, I, P, P, P, P, P, P, P, F, L, I, I, I, I, F, I, P]),
-    "aphro_latent_attention_plain": (I, [P, L, L, P, L, L, P, L, L, P, P, I, L, I, P, P, P, P, F, L, I, I, I, I, F, I, P, I, P]),
+    "aphro_latent_attention_plain": (I, [P, L, L, P, L, L, P, L, L, P, P, I, L, I, P, P, P, P, F, L, I, I, I, I, F, I, P, P, L, I, P]),
     "aphro_latent_attention_fast_supported": (I, [I, I, I, I]),
     "aphro_latent_attention_splits": (I, [L, I, I, I, I]),
-    "aphro_latent_attention": (I, [P, L, L, P, L, L, P, L, L, P, P, I, L, I, P, P, P, P, P, F, L, I, I, I, I, I, I, I, F, I, P, P, L, I, P]),
+    "aphro_latent_attention": (I, [P, L, L, P, L, L, P, L, L, P, P, I, L, I, P, P, P, P, P, F, L, I, I, I, I, I, I, I, F, I, P, P, L, P, L, I, P]),
     "aphro_sigmoid_gate_mul": (I, [P, L, P, L, P, L, L, I, I, P]),
     "aphro_experts_route_grouped": (I, [P, P, P, L, I, I, I, I, I, F, P]),
     "aphro_experts_route_topk": (I, [P, P, P, P, L, I, I, P]),
@@ -210,7 +210,11 @@ MIXERS_SIGNATURES = {
     "aphro_logit_softcap": (I, [P, P, L, F, F, I, P]),
     "aphro_gated_delta_scan": (I, [P, P, L, P, L, P, L, P, L, P, L, P, P, P, P, I, P, P, P, I, L, I, I, I, I, I, F, F, I, I, P]),
     "aphro_gated_head_rms_norm": (I, [P, L, P, P, P, L, L, I, I, F, I, I, P]),
-    "aphro_rotary_qk_norm_kv_write": (I, [P, L, P, P, P, L, P, L, P, L, P, L, P, L, F, P, P, P, P, L, I, I, I, I, I, I, I, P, P, F, I, P]),
+    "aphro_conv_rotary_supported": (I, [I, I, I]),
+    "aphro_conv_rotary_qk_norm_kv_write": (I, [P, L, P, P, P, L, P, L, P, P, P, P, P, P, P, P, F, P, P, F, L, I, I, I, I, I, I, I, I, I, P]),
+    "aphro_short_conv_state": (I, [P, P, L, P, P, P, P, I, I, I, I, P]),
+    "aphro_residual_tanh_norm": (I, [P, I, P, L, P, L, P, P, L, F, P, P, P, F, P, P, P, L, I, I, P]),
+    "aphro_rotary_qk_norm_kv_write": (I, [P, L, P, P, P, L, P, L, P, L, P, L, P, L, F, P, P, P, P, F, L, I, I, I, I, I, I, I, P, P, F, I, P]),
 }
 
 OK = 0

@@ -10,7 +10,8 @@
 //                      of the shared key part at the token's position -> the cache row at its slot
 //   latent_attention   any sizes, fp32 math: a workgroup of four waves per (row, head); lane = key for the scores, lane =
 //                      column for P C; rotates the query's rotary part on load; optional sliding window (row i sees key j
-//                      with 0 <= i - j < window) and per-head sink (exp(sink) joins the softmax denominator, unscaled)
+//                      with 0 <= i - j < window), per-head sink (exp(sink) joins the softmax denominator, unscaled) and
+//                      per-head output gate (sigmoid of one number per row and head)
 //   sigmoid_gate_mul   out = x * sigmoid(gate), elementwise
 // Rotation ("rotate half" over the first rot_dims numbers of the rotary part): the pair (u, v) = (x[i], x[i + rot_dims / 2])
 // becomes (u cos a - v sin a, v cos a + u sin a) * mscale with a = position * inv_freq[i], all in fp32.
@@ -108,7 +109,8 @@ __global__ __launch_bounds__(256) void latent_attention_kernel(
     const typename T::storage* __restrict__ cache, const int32_t* __restrict__ block_tables, int max_blocks, int64_t num_blocks,
     int block_size, const int32_t* __restrict__ q_start, const int32_t* __restrict__ ctx_len,
     const int32_t* __restrict__ seq_of_token, const float* __restrict__ inv_freq, float mscale, int kv_rank, int rot_dim,
-    int rot_dims, float scale, int window, const float* __restrict__ sink) {
+    int rot_dims, float scale, int window, const float* __restrict__ sink, const typename T::storage* __restrict__ gate,
+    int64_t gate_stride) {
   __shared__ __attribute__((aligned(16))) float qsh[LA_MAX_DIM];
   __shared__ float merge[LA_WAVES][2 + EPL * 64];
   const int t = blockIdx.x, h = blockIdx.y;
@@ -187,7 +189,8 @@ __global__ __launch_bounds__(256) void latent_attention_kernel(
     f[w] = (merge[w][0] == -INFINITY) ? 0.f : expf(merge[w][0] - M);
     L += merge[w][1] * f[w];
   }
-  const float inv = 1.0f / L;
+  float inv = 1.0f / L;
+  if (gate) inv *= sigmoid_f(T::to_f32(gate[(int64_t)t * gate_stride + h]));
 #pragma unroll
   for (int c = 0; c < EPL; ++c) {
     const int col = lane + 64 * c;
@@ -271,7 +274,7 @@ extern "C" int aphro_latent_attention_plain(void* out, int64_t out_stride, int64
                                             int64_t num_blocks, int block_size, const int32_t* q_start, const int32_t* ctx_len,
                                             const int32_t* seq_of_token, const float* inv_freq, float mscale, int64_t num_tokens,
                                             int heads, int kv_rank, int rot_dim, int rot_dims, float scale, int window,
-                                            const float* sink, int dtype, void* stream) {
+                                            const float* sink, const void* gate, int64_t gate_stride, int dtype, void* stream) {
   if (num_tokens == 0) return APHRO_OK;
   APHRO_CHECK(out && q_lat && (q_rot || rot_dim == 0) && cache && block_tables && q_start && ctx_len && seq_of_token &&
                   (rot_dims == 0 || inv_freq), "latent_attention: null argument");
@@ -280,13 +283,14 @@ extern "C" int aphro_latent_attention_plain(void* out, int64_t out_stride, int64
               "latent_attention: %d heads, rank %d (<= %d), rotary part %d of which %d rotate", heads, kv_rank, 64 * LA_MAX_EPL,
               rot_dim, rot_dims);
   APHRO_CHECK(block_size > 0 && max_blocks > 0 && num_blocks > 0, "latent_attention: bad cache geometry");
+  APHRO_CHECK(!gate || gate_stride >= heads, "latent_attention: gate rows hold one number per head");
   const dim3 grid((unsigned)num_tokens, (unsigned)heads);
   const int epl = (kv_rank + 63) / 64;
 #define LA_LAUNCH(EPL)                                                                                                         \
   hipLaunchKernelGGL((latent_attention_kernel<T, EPL>), grid, dim3(256), 0, (hipStream_t)stream, (S*)out, out_stride,           \
                      out_head_stride, (const S*)q_lat, ql_stride, ql_head_stride, (const S*)q_rot, qr_stride, qr_head_stride,   \
                      (const S*)cache, block_tables, max_blocks, num_blocks, block_size, q_start, ctx_len, seq_of_token, inv_freq, \
-                     mscale, kv_rank, rot_dim, rot_dims, scale, window, sink)
+                     mscale, kv_rank, rot_dim, rot_dims, scale, window, sink, (const S*)gate, gate_stride)
   MIX_DISPATCH_DTYPE(dtype, {
     typedef typename T::storage S;
     switch (epl) {

@@ -29,6 +29,8 @@ struct LAParams {
   const int32_t* ctx_len;
   const float* inv_freq;
   const float* sink;  // fp32 [heads] or NULL
+  const uint16_t* gate;      // raw, one number per row and head (row stride gate_stride), or NULL: sigmoid of it scales the head's output
+  int64_t gate_stride;
   int window;         // <= 0: none
   int64_t out_stride, out_head_stride, ql_stride, ql_head_stride, qr_stride, qr_head_stride, num_blocks;
   int max_blocks, block_size, bs_shift, heads, nsplit;
@@ -288,6 +290,7 @@ __global__ __launch_bounds__(LF_THREADS) void la_mfma_kernel(LAParams p) {
       const float s2 = p.sink[head] * LOG2E, M = fmaxf(m_run, s2), fo = __builtin_amdgcn_exp2f(m_run - M);
       f = fo / (l * fo + __builtin_amdgcn_exp2f(s2 - M));
     }
+    if (p.gate) f *= sigmoid_f(BFloat::to_f32(p.gate[(int64_t)(s0 + tok) * p.gate_stride + head]));
     uint16_t* op = p.out + (int64_t)(s0 + tok) * p.out_stride + (int64_t)head * p.out_head_stride + 16 * G::NDH * half;
 #pragma unroll
     for (int dt = 0; dt < G::NDH; ++dt)
@@ -309,7 +312,8 @@ __global__ __launch_bounds__(LF_THREADS) void la_mfma_kernel(LAParams p) {
 // split's piece in flight before it adds them up
 constexpr int LA_MAX_SPLIT = 16;
 __global__ void la_merge_kernel(uint16_t* __restrict__ out, int64_t out_stride, int64_t out_head_stride, const float* __restrict__ ws,
-                                int heads, int nsplit, int R, const float* __restrict__ sink) {
+                                int heads, int nsplit, int R, const float* __restrict__ sink, const uint16_t* __restrict__ gate,
+                                int64_t gate_stride) {
   const int64_t t = blockIdx.x;
   const int head = blockIdx.y;
   const float* wp = ws + ((t * heads + head) * nsplit) * (int64_t)(2 + R);
@@ -335,7 +339,8 @@ __global__ void la_merge_kernel(uint16_t* __restrict__ out, int64_t out_stride, 
       a0 += v[zz][0] * f;
       a1 += v[zz][1] * f;
     }
-  const float inv = L > 0.f ? 1.f / L : 0.f;
+  float inv = L > 0.f ? 1.f / L : 0.f;
+  if (gate) inv *= sigmoid_f(BFloat::to_f32(gate[t * gate_stride + head]));
   if (col < R)
     *reinterpret_cast<uint32_t*>(out + t * out_stride + (int64_t)head * out_head_stride + col) = pack2_16<true>(a0 * inv, a1 * inv);
 }
@@ -358,7 +363,7 @@ static int la_launch(const LAParams& p, int num_seqs, int max_q_len, int64_t num
                      stream, p);
   if (p.nsplit > 1)
     hipLaunchKernelGGL(la_merge_kernel, dim3((unsigned)num_tokens, (unsigned)p.heads), dim3((R / 2 + 63) / 64 * 64), 0, stream, p.out,
-                       p.out_stride, p.out_head_stride, p.ws, p.heads, p.nsplit, R, p.sink);
+                       p.out_stride, p.out_head_stride, p.ws, p.heads, p.nsplit, R, p.sink, p.gate, p.gate_stride);
   return APHRO_OK;
 }
 
@@ -372,9 +377,10 @@ extern "C" int aphro_latent_attention_plain(void* out, int64_t out_stride, int64
                                             int64_t num_blocks, int block_size, const int32_t* q_start, const int32_t* ctx_len,
                                             const int32_t* seq_of_token, const float* inv_freq, float mscale, int64_t num_tokens,
                                             int heads, int kv_rank, int rot_dim, int rot_dims, float scale, int window,
-                                            const float* sink, int dtype, void* stream);
+                                            const float* sink, const void* gate, int64_t gate_stride, int dtype, void* stream);
 
-#define LA_FAST_SIZES(X) X(128, 16) X(128, 32) X(256, 32) X(256, 64) X(512, 64)
+#define LA_FAST_SIZES(X) \
+  X(64, 0) X(96, 0) X(128, 0) X(128, 16) X(128, 32) X(192, 0) X(256, 0) X(256, 32) X(256, 64) X(384, 0) X(512, 0) X(512, 64)
 
 extern "C" int aphro_latent_attention_fast_supported(int kv_rank, int rot_dim, int rot_dims, int dtype) {
   if (dtype != APHRO_BF16 || rot_dims != rot_dim) return 0;
@@ -402,8 +408,8 @@ extern "C" int aphro_latent_attention(void* out, int64_t out_stride, int64_t out
                                       int block_size, const int32_t* q_start, const int32_t* q_len, const int32_t* ctx_len,
                                       const int32_t* seq_of_token, const float* inv_freq, float mscale, int64_t num_tokens,
                                       int num_seqs, int max_q_len, int max_kv_len, int heads, int kv_rank, int rot_dim, int rot_dims,
-                                      float scale, int window, const float* sink, float* workspace, int64_t workspace_floats,
-                                      int dtype, void* stream) {
+                                      float scale, int window, const float* sink, const void* gate, int64_t gate_stride, float* workspace,
+                                      int64_t workspace_floats, int dtype, void* stream) {
   if (num_tokens == 0) return APHRO_OK;
   const auto al16 = [](const void* ptr) { return ((uintptr_t)ptr & 15) == 0; };
   const bool fast = aphro_latent_attention_fast_supported(kv_rank, rot_dim, rot_dims, dtype) && q_len && num_seqs > 0 && max_q_len > 0 &&
@@ -414,8 +420,9 @@ extern "C" int aphro_latent_attention(void* out, int64_t out_stride, int64_t out
     return aphro_latent_attention_plain(out, out_stride, out_head_stride, q_lat, ql_stride, ql_head_stride, q_rot, qr_stride,
                                         qr_head_stride, cache, block_tables, max_blocks, num_blocks, block_size, q_start, ctx_len,
                                         seq_of_token, inv_freq, mscale, num_tokens, heads, kv_rank, rot_dim, rot_dims, scale, window,
-                                        sink, dtype, stream);
-  APHRO_CHECK(out && q_lat && q_rot && cache && block_tables && q_start && ctx_len && inv_freq, "latent_attention: null argument");
+                                        sink, gate, gate_stride, dtype, stream);
+  APHRO_CHECK(!gate || gate_stride >= heads, "latent_attention: gate rows hold one number per head");
+  APHRO_CHECK(out && q_lat && (q_rot || rot_dim == 0) && cache && block_tables && q_start && ctx_len && (inv_freq || rot_dim == 0), "latent_attention: null argument");
   APHRO_CHECK(heads > 0 && heads <= 65535 && block_size > 0 && max_blocks > 0 && num_blocks > 0 && num_seqs <= 65535,
               "latent_attention: bad geometry");
   LAParams p;
@@ -429,6 +436,8 @@ extern "C" int aphro_latent_attention(void* out, int64_t out_stride, int64_t out
   p.ctx_len = ctx_len;
   p.inv_freq = inv_freq;
   p.sink = sink;
+  p.gate = (const uint16_t*)gate;
+  p.gate_stride = gate_stride;
   p.window = window;
   p.out_stride = out_stride;
   p.out_head_stride = out_head_stride;

@@ -190,7 +190,7 @@ __global__ void residual_layer_norm_vec8_kernel(float* __restrict__ residual, co
 }
 
 template <typename T, int ACT>
-__global__ void act_and_mul_vec8_kernel(typename T::storage* __restrict__ out, const typename T::storage* __restrict__ in,
+__global__ void act_and_mul_vec8_kernel(typename T::storage* __restrict__ out, int64_t out_stride, const typename T::storage* __restrict__ in,
                                         int64_t in_stride, int d) {
   const int64_t t = blockIdx.y;
   const int i0 = (blockIdx.x * blockDim.x + threadIdx.x) * 8;
@@ -200,15 +200,15 @@ __global__ void act_and_mul_vec8_kernel(typename T::storage* __restrict__ out, c
   load8<T>(in + t * in_stride + d + i0, u);
 #pragma unroll
   for (int j = 0; j < 8; ++j) g[j] = (ACT == 0 ? silu_f(g[j]) : gelu_tanh_f(g[j])) * u[j];
-  store8<T>(out + t * (int64_t)d + i0, g);
+  store8<T>(out + t * out_stride + i0, g);
 }
 
 template <typename T, int ACT>
-__global__ void act_and_mul_kernel(typename T::storage* __restrict__ out, const typename T::storage* __restrict__ in,
+__global__ void act_and_mul_kernel(typename T::storage* __restrict__ out, int64_t out_stride, const typename T::storage* __restrict__ in,
                                    int64_t in_stride, int d) {
   const int64_t t = blockIdx.x;
   const typename T::storage* a = in + t * in_stride;
-  typename T::storage* o = out + t * (int64_t)d;
+  typename T::storage* o = out + t * out_stride;
   for (int i = threadIdx.x; i < d; i += blockDim.x) {
     const float g = T::to_f32(a[i]), u = T::to_f32(a[d + i]);
     o[i] = T::from_f32((ACT == 0 ? silu_f(g) : gelu_tanh_f(g)) * u);
@@ -399,19 +399,19 @@ extern "C" int aphro_residual_layer_norm(float* residual, const void* y, int64_t
   return APHRO_OK;
 }
 
-extern "C" int aphro_act_and_mul(void* out, const void* in, int64_t in_stride, int64_t num_tokens, int d, int act, int dtype,
+extern "C" int aphro_act_and_mul(void* out, int64_t out_stride, const void* in, int64_t in_stride, int64_t num_tokens, int d, int act, int dtype,
                                  void* stream) {
   if (num_tokens == 0) return APHRO_OK;
-  APHRO_CHECK(out && in && d > 0 && in_stride >= 2 * (int64_t)d && (act == 0 || act == 1), "act_and_mul: bad arguments");
-  if ((d & 7) == 0 && (in_stride & 7) == 0 && ((uintptr_t)in & 15) == 0 && ((uintptr_t)out & 15) == 0 && num_tokens <= 65535) {
+  APHRO_CHECK(out && in && d > 0 && in_stride >= 2 * (int64_t)d && out_stride >= d && (act == 0 || act == 1), "act_and_mul: bad arguments");
+  if ((d & 7) == 0 && (in_stride & 7) == 0 && (out_stride & 7) == 0 && ((uintptr_t)in & 15) == 0 && ((uintptr_t)out & 15) == 0 && num_tokens <= 65535) {
     const int per_row = d / 8, threads = per_row >= 256 ? 256 : (per_row + 63) / 64 * 64;
     const dim3 grid((unsigned)((per_row + threads - 1) / threads), (unsigned)num_tokens);
     MIX_DISPATCH_DTYPE(dtype, {
       typedef typename T::storage S;
       if (act == 0)
-        hipLaunchKernelGGL((act_and_mul_vec8_kernel<T, 0>), grid, dim3(threads), 0, (hipStream_t)stream, (S*)out, (const S*)in, in_stride, d);
+        hipLaunchKernelGGL((act_and_mul_vec8_kernel<T, 0>), grid, dim3(threads), 0, (hipStream_t)stream, (S*)out, out_stride, (const S*)in, in_stride, d);
       else
-        hipLaunchKernelGGL((act_and_mul_vec8_kernel<T, 1>), grid, dim3(threads), 0, (hipStream_t)stream, (S*)out, (const S*)in, in_stride, d);
+        hipLaunchKernelGGL((act_and_mul_vec8_kernel<T, 1>), grid, dim3(threads), 0, (hipStream_t)stream, (S*)out, out_stride, (const S*)in, in_stride, d);
     });
     APHRO_LAUNCH_CHECK();
     return APHRO_OK;
@@ -420,10 +420,10 @@ extern "C" int aphro_act_and_mul(void* out, const void* in, int64_t in_stride, i
     typedef typename T::storage S;
     if (act == 0)
       hipLaunchKernelGGL((act_and_mul_kernel<T, 0>), dim3((unsigned)num_tokens), dim3(block_for(d)), 0, (hipStream_t)stream,
-                         (S*)out, (const S*)in, in_stride, d);
+                         (S*)out, out_stride, (const S*)in, in_stride, d);
     else
       hipLaunchKernelGGL((act_and_mul_kernel<T, 1>), dim3((unsigned)num_tokens), dim3(block_for(d)), 0, (hipStream_t)stream,
-                         (S*)out, (const S*)in, in_stride, d);
+                         (S*)out, out_stride, (const S*)in, in_stride, d);
   });
   APHRO_LAUNCH_CHECK();
   return APHRO_OK;

@@ -1,10 +1,10 @@
 // What happens between the input product [q | k | v] of a rotary grouped-query attention and its paged cache, in one launch:
 //   * the first rot_dims numbers of every query and key head are turned by position * inv_freq[i] -- layout 0 pairs number i
 //     with number i + rot_dims / 2 ("rotate half"), layout 1 pairs number 2 i with number 2 i + 1 (interleaved); the pair
-//     (u, v) becomes (u cos a - v sin a, v cos a + u sin a); the rest of the head passes unchanged;
+//     (u, v) becomes (u cos a - v sin a, v cos a + u sin a), cos and sin times mscale; the rest of the head passes unchanged;
 //   * optionally every query and key head is divided by its root mean square over the head, with a weight per number of the
 //     head (one for queries, one for keys, shared by their heads) or without.  The weight acts before the rotation; the
-//     statistic does not depend on the order, since a rotation keeps every pair's length;
+//     statistic is taken before it too;
 //   * optionally the values are blended with another tensor's values of the same tokens, v <- (1 - lambda) v + lambda v_other;
 //   * queries go to a dense output, keys and values into the token-major paged caches at the rows' slots.
 // Positions, angles, cos / sin, the statistics and the blend are fp32; one rounding to the storage type.
@@ -23,7 +23,7 @@ __global__ __launch_bounds__(256) void rotary_qk_norm_kv_write_kernel(
     const typename T::storage* __restrict__ q, int64_t q_stride, const typename T::storage* __restrict__ k, int64_t k_stride,
     const typename T::storage* __restrict__ v, int64_t v_stride, const typename T::storage* __restrict__ v_other,
     int64_t v_other_stride, float lambda, const int32_t* __restrict__ q_start, const int32_t* __restrict__ ctx_len,
-    const int32_t* __restrict__ seq_of_token, const float* __restrict__ inv_freq, int heads, int kv_heads, int dim, int vdim,
+    const int32_t* __restrict__ seq_of_token, const float* __restrict__ inv_freq, float mscale, int heads, int kv_heads, int dim, int vdim,
     int rot_dims, int layout, int qk_norm, const typename T::storage* __restrict__ q_weight,
     const typename T::storage* __restrict__ k_weight, float eps) {
   const int64_t t = blockIdx.x;
@@ -77,6 +77,8 @@ __global__ __launch_bounds__(256) void rotary_qk_norm_kv_write_kernel(
         }
         float c, sn;
         sincosf(pos * inv_freq[f], &sn, &c);
+        c *= mscale;
+        sn *= mscale;
         float other = T::to_f32(src[partner]);
         if (nw) other *= T::to_f32(nw[partner]);
         x = first ? x * c - other * sn : x * c + other * sn;
@@ -131,7 +133,7 @@ __global__ __launch_bounds__(256) void rotary_qk_norm_kv_write_vec8_kernel(
     const typename T::storage* __restrict__ q, int64_t q_stride, const typename T::storage* __restrict__ k, int64_t k_stride,
     const typename T::storage* __restrict__ v, int64_t v_stride, const typename T::storage* __restrict__ v_other,
     int64_t v_other_stride, float lambda, const int32_t* __restrict__ q_start, const int32_t* __restrict__ ctx_len,
-    const int32_t* __restrict__ seq_of_token, const float* __restrict__ inv_freq, int heads, int kv_heads, int dim, int vdim,
+    const int32_t* __restrict__ seq_of_token, const float* __restrict__ inv_freq, float mscale, int heads, int kv_heads, int dim, int vdim,
     int rot_dims, int layout, int qk_norm, const typename T::storage* __restrict__ q_weight,
     const typename T::storage* __restrict__ k_weight, float eps, int tph) {
   const int64_t t = blockIdx.x;
@@ -193,6 +195,8 @@ __global__ __launch_bounds__(256) void rotary_qk_norm_kv_write_vec8_kernel(
         for (int e = 0; e < 8; ++e) {
           float c, sn;
           sincosf(pos * inv_freq[f0 + e], &sn, &c);
+          c *= mscale;
+          sn *= mscale;
           x[e] = first ? x[e] * c - o[e] * sn : x[e] * c + o[e] * sn;
         }
       } else {
@@ -200,6 +204,8 @@ __global__ __launch_bounds__(256) void rotary_qk_norm_kv_write_vec8_kernel(
         for (int e = 0; e < 8; e += 2) {
           float c, sn;
           sincosf(pos * inv_freq[(i0 + e) >> 1], &sn, &c);
+          c *= mscale;
+          sn *= mscale;
           const float a = x[e], b = x[e + 1];
           x[e] = a * c - b * sn;
           x[e + 1] = b * c + a * sn;
@@ -301,7 +307,7 @@ extern "C" int aphro_rotary_qk_norm_kv_write(void* q_out, int64_t q_out_stride, 
                                              int64_t num_cache_rows, const void* q, int64_t q_stride, const void* k, int64_t k_stride,
                                              const void* v, int64_t v_stride, const void* v_other, int64_t v_other_stride, float lambda,
                                              const int32_t* q_start, const int32_t* ctx_len, const int32_t* seq_of_token,
-                                             const float* inv_freq, int64_t num_tokens, int heads, int kv_heads, int dim, int vdim,
+                                             const float* inv_freq, float mscale, int64_t num_tokens, int heads, int kv_heads, int dim, int vdim,
                                              int rot_dims, int layout, int qk_norm, const void* q_weight, const void* k_weight, float eps, int dtype, void* stream) {
   if (num_tokens == 0) return APHRO_OK;
   APHRO_CHECK(q_out && k_cache && v_cache && slot_mapping && q && k && v && q_start && ctx_len && seq_of_token && (rot_dims == 0 || inv_freq),
@@ -328,13 +334,13 @@ extern "C" int aphro_rotary_qk_norm_kv_write(void* q_out, int64_t q_out_stride, 
       hipLaunchKernelGGL((rotary_qk_norm_kv_write_vec8_kernel<T>), dim3((unsigned)num_tokens, (unsigned)((units + per_block - 1) / per_block)),
                          dim3(256), 0, (hipStream_t)stream, (S*)q_out, q_out_stride, (S*)k_cache, (S*)v_cache, slot_mapping, num_cache_rows,
                          (const S*)q, q_stride, (const S*)k, k_stride, (const S*)v, v_stride, (const S*)v_other, v_other_stride, lambda,
-                         q_start, ctx_len, seq_of_token, inv_freq, heads, kv_heads, dim, vdim, rot_dims, layout, qk_norm,
+                         q_start, ctx_len, seq_of_token, inv_freq, mscale, heads, kv_heads, dim, vdim, rot_dims, layout, qk_norm,
                          (const S*)q_weight, (const S*)k_weight, eps, tph);
     } else
     hipLaunchKernelGGL((rotary_qk_norm_kv_write_kernel<T>), dim3((unsigned)num_tokens, (unsigned)((units + 3) / 4)), dim3(256), 0,
                        (hipStream_t)stream, (S*)q_out, q_out_stride, (S*)k_cache, (S*)v_cache, slot_mapping, num_cache_rows, (const S*)q,
                        q_stride, (const S*)k, k_stride, (const S*)v, v_stride, (const S*)v_other, v_other_stride, lambda, q_start,
-                       ctx_len, seq_of_token, inv_freq, heads, kv_heads, dim, vdim, rot_dims, layout, qk_norm, (const S*)q_weight,
+                       ctx_len, seq_of_token, inv_freq, mscale, heads, kv_heads, dim, vdim, rot_dims, layout, qk_norm, (const S*)q_weight,
                        (const S*)k_weight, eps);
   });
   APHRO_LAUNCH_CHECK();

@@ -184,6 +184,20 @@ __global__ void short_conv_state_kernel(typename T::storage* __restrict__ state,
 
 using namespace aphro;
 
+extern "C" int aphro_short_conv_state(void* state, const void* u, int64_t u_stride, const int32_t* state_slots, const int32_t* q_start,
+                                      const int32_t* q_len, const int32_t* ctx_len, int num_seqs, int channels, int taps, int dtype,
+                                      void* stream) {
+  APHRO_CHECK(state && u && state_slots && q_start && q_len && ctx_len && num_seqs > 0 && channels > 0 && (channels + 255) / 256 <= 65535 &&
+                  u_stride >= channels && taps >= 2 && taps <= SC_MAX_TAPS, "short_conv_state: bad arguments (%d taps)", taps);
+  MIX_DISPATCH_DTYPE(dtype, {
+    typedef typename T::storage S;
+    hipLaunchKernelGGL((short_conv_state_kernel<T>), dim3((unsigned)num_seqs, (unsigned)((channels + 255) / 256)), dim3(256), 0,
+                       (hipStream_t)stream, (S*)state, (const S*)u, u_stride, state_slots, q_start, q_len, ctx_len, channels, taps);
+  });
+  APHRO_LAUNCH_CHECK();
+  return APHRO_OK;
+}
+
 extern "C" int aphro_short_conv(void* q_out, int64_t q_out_stride, void* k_cache, void* v_cache, const int64_t* cache_slots,
                                 int64_t num_cache_slots, const void* u, int64_t u_stride, const void* w, const void* bias,
                                 void* state,
@@ -220,11 +234,9 @@ extern "C" int aphro_short_conv(void* q_out, int64_t q_out_stride, void* k_cache
                        (hipStream_t)stream, (S*)q_out, q_out_stride, (S*)k_cache, (S*)v_cache, cache_slots, num_cache_slots,
                        (const S*)u, u_stride, (const S*)w, (const S*)bias, (const S*)state, state_slots, q_start, ctx_len, seq_of_token, cq, ck,
                        cv, taps, act);
-    if (taps > 1)
-      hipLaunchKernelGGL((short_conv_state_kernel<T>), dim3((unsigned)num_seqs, (unsigned)((C + 255) / 256)), dim3(256), 0,
-                         (hipStream_t)stream, (S*)state, (const S*)u, u_stride, state_slots, q_start, q_len, ctx_len, C, taps);
   });
 #undef SC_VEC
   APHRO_LAUNCH_CHECK();
-  return APHRO_OK;
+  if (taps == 1) return APHRO_OK;
+  return aphro_short_conv_state(state, u, u_stride, state_slots, q_start, q_len, ctx_len, num_seqs, C, taps, dtype, stream);
 }

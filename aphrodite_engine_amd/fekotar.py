@@ -207,9 +207,7 @@ class FekotarForCausalLM(nn.Module):
                 return mix.uq.weight_loader(mix.uq.weight, t.to(mix.uq.weight.dtype), 0)
             if key == "o":
                 return mix.out_proj.weight_loader(mix.out_proj.weight, t.to(mix.out_proj.weight.dtype), 0)
-            if key == "uk":
-                return put(mix.w_uk.data.view(mix.heads * mix.dim, mix.kv_rank), t, name)
-            return put(mix.w_uv.data.view(mix.heads * mix.vdim, mix.kv_rank), t, name)
+            return mix.load_up_projection(key, t, name)
         key, m = rest[4:], layer.mlp
         if isinstance(m, ClampedGLUMLP):
             part, is_bias = (key[:-2], True) if key.endswith(".b") else (key, False)

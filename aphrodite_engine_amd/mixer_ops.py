@@ -145,13 +145,15 @@ def silu_gate_part_rms_norm(out: torch.Tensor, x: torch.Tensor, gate: torch.Tens
         weight.data_ptr(), T, N, N // parts, float(eps), float(out_scale), _dt(out), _stream()), "silu_gate_part_rms_norm")
 
 
-def act_and_mul(x: torch.Tensor, act: int) -> torch.Tensor:
-    """[T, 2 d] -> [T, d]: act(x[:, :d]) * x[:, d:]."""
-    _cuda(x)
+def act_and_mul(x: torch.Tensor, act: int, out: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """[T, 2 d] -> [T, d]: act(x[:, :d]) * x[:, d:], into ``out`` (dense rows, any row stride) if given."""
+    _cuda(x, out)
     _need(x.dim() == 2 and x.shape[1] % 2 == 0, "act_and_mul: [T, 2 d]")
     d = x.shape[1] // 2
-    out = torch.empty(x.shape[0], d, dtype=x.dtype, device=x.device)
-    check(_lib.mixers_lib().aphro_act_and_mul(out.data_ptr(), x.data_ptr(), _rows(x, 2 * d, "act_and_mul"), x.shape[0], d,
+    if out is None:
+        out = torch.empty(x.shape[0], d, dtype=x.dtype, device=x.device)
+    _need(out.dtype == x.dtype and out.shape == (x.shape[0], d), "act_and_mul: out [T, d] of x's dtype")
+    check(_lib.mixers_lib().aphro_act_and_mul(out.data_ptr(), _rows(out, d, "act_and_mul out"), x.data_ptr(), _rows(x, 2 * d, "act_and_mul"), x.shape[0], d,
                                               int(act), _dt(x), _stream()), "act_and_mul")
     return out
 
@@ -644,15 +646,15 @@ def latent_attention(out: torch.Tensor, q_lat: torch.Tensor, q_rot: Optional[tor
                      block_tables: torch.Tensor, q_start: torch.Tensor, q_len: torch.Tensor, ctx_len: torch.Tensor,
                      seq_of_token: torch.Tensor, q_len_range, inv_freq: Optional[torch.Tensor], mscale: float, rot_dims: int,
                      scale: float, max_kv_len: int = 0, plain: bool = False, window: int = 0,
-                     sink: Optional[torch.Tensor] = None) -> None:
+                     sink: Optional[torch.Tensor] = None, gate: Optional[torch.Tensor] = None) -> None:
     """Causal softmax attention of a batch of segments over latent cache rows [c | k_r] that all heads share.  q_lat
     [T, heads, kv_rank] (every head's query carried into the latent), q_rot [T, heads, rot_dim] (raw: rotated here at the row's
     position), out [T, heads, kv_rank] = sum_j p_ij c_j -- any strides over tokens and heads.  ``q_len_range`` (shortest, longest
     segment) and ``max_kv_len`` (longest ctx_len + q_len), known on the host, choose the work split of the matrix-core kernel,
     which serves the sizes ``latent_attention_fast_supported`` names; ``plain`` forces the fp32-math kernel of any size.
     ``window`` > 0: a row sees only the last ``window`` keys up to its own; ``sink`` fp32 [heads]: exp(sink) joins every row's
-    softmax denominator (unscaled, without a value)."""
-    _cuda(out, q_lat, q_rot, cache, block_tables, q_start, q_len, ctx_len, seq_of_token, inv_freq, sink)
+    softmax denominator (unscaled, without a value); ``gate`` [T, heads] raw: a head's output times sigmoid of its number."""
+    _cuda(out, q_lat, q_rot, cache, block_tables, q_start, q_len, ctx_len, seq_of_token, inv_freq, sink, gate)
     _need(sink is None or (sink.dtype == torch.float32 and sink.is_contiguous() and sink.numel() == q_lat.shape[1]),
           "latent_attention: sink fp32 [heads]")
     window = max(int(window), 0)
@@ -660,6 +662,10 @@ def latent_attention(out: torch.Tensor, q_lat: torch.Tensor, q_rot: Optional[tor
     nb, bs, D = cache.shape
     P_ = D - R
     S = q_start.numel()
+    gs = 0
+    if gate is not None:
+        _need(gate.dtype == q_lat.dtype and gate.shape == (T, H), "latent_attention: gate [T, heads] of the activation dtype")
+        gs = _rows(gate, H, "latent_attention gate")
     _need(cache.is_contiguous() and cache.dtype == q_lat.dtype == out.dtype and P_ >= 0, "latent_attention: cache [blocks, block, rank + rot]")
     os_, ohs = _head_view(out, T, H, R, "latent_attention out")
     qs, qhs = _head_view(q_lat, T, H, R, "latent_attention q_lat")
@@ -679,7 +685,7 @@ def latent_attention(out: torch.Tensor, q_lat: torch.Tensor, q_rot: Optional[tor
         check(lib.aphro_latent_attention_plain(
             out.data_ptr(), os_, ohs, q_lat.data_ptr(), qs, qhs, _p(q_rot), rs, rhs, cache.data_ptr(), block_tables.data_ptr(),
             block_tables.shape[1], nb, bs, q_start.data_ptr(), ctx_len.data_ptr(), seq_of_token.data_ptr(), _p(inv_freq), float(mscale),
-            T, H, R, P_, int(rot_dims), float(scale), window, _p(sink), _dt(q_lat), _stream()), "latent_attention")
+            T, H, R, P_, int(rot_dims), float(scale), window, _p(sink), _p(gate), gs, _dt(q_lat), _stream()), "latent_attention")
         return
     lo, hi = int(q_len_range[0]), int(q_len_range[1])
     _need(0 < lo <= hi, "latent_attention: q_len_range (shortest, longest)")
@@ -694,8 +700,8 @@ def latent_attention(out: torch.Tensor, q_lat: torch.Tensor, q_rot: Optional[tor
     check(lib.aphro_latent_attention(
         out.data_ptr(), os_, ohs, q_lat.data_ptr(), qs, qhs, _p(q_rot), rs, rhs, cache.data_ptr(), block_tables.data_ptr(),
         block_tables.shape[1], nb, bs, q_start.data_ptr(), q_len.data_ptr(), ctx_len.data_ptr(), seq_of_token.data_ptr(), _p(inv_freq),
-        float(mscale), T, S, hi, int(max_kv_len), H, R, P_, int(rot_dims), float(scale), window, _p(sink), _p(ws), ws_n, _dt(q_lat),
-        _stream()), "latent_attention")
+        float(mscale), T, S, hi, int(max_kv_len), H, R, P_, int(rot_dims), float(scale), window, _p(sink), _p(gate), gs, _p(ws), ws_n,
+        _dt(q_lat), _stream()), "latent_attention")
 
 
 def latent_attention_fast_supported(kv_rank: int, rot_dim: int, rot_dims: int, dtype: torch.dtype) -> bool:
@@ -870,9 +876,10 @@ def rotary_qk_norm_kv_write(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, k
                             slot_mapping: torch.Tensor, q_start: torch.Tensor, ctx_len: torch.Tensor, seq_of_token: torch.Tensor,
                             inv_freq: Optional[torch.Tensor], rot_dims: int, layout: int = ROTARY_HALF, qk_norm: bool = False,
                             eps: float = 1e-6, v_other: Optional[torch.Tensor] = None, lam: float = 0.0,
-                            q_weight: Optional[torch.Tensor] = None, k_weight: Optional[torch.Tensor] = None) -> torch.Tensor:
+                            q_weight: Optional[torch.Tensor] = None, k_weight: Optional[torch.Tensor] = None,
+                            mscale: float = 1.0) -> torch.Tensor:
     """q [T, heads * dim], k [T, kv_heads * dim], v [T, kv_heads * vdim] (dense rows of one input product): rotates the first
-    ``rot_dims`` numbers of every q and k head at the row's position, optionally brings every q and k head to unit RMS (times ``q_weight`` /
+    ``rot_dims`` numbers of every q and k head at the row's position (cos and sin times ``mscale``), optionally brings every q and k head to unit RMS (times ``q_weight`` /
     ``k_weight`` [dim], applied before the rotation), blends v
     with ``v_other`` ((1 - lam) v + lam v_other), writes k and v into the paged caches k_cache [blocks, block, kv_heads, dim] /
     v_cache [.., vdim] at ``slot_mapping`` and returns the prepared queries [T, heads * dim]."""
@@ -901,7 +908,7 @@ def rotary_qk_norm_kv_write(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, k
     check(_lib.mixers_lib().aphro_rotary_qk_norm_kv_write(
         q_out.data_ptr(), H * d, k_cache.data_ptr(), v_cache.data_ptr(), slot_mapping.data_ptr(), nb * bs, q.data_ptr(),
         _rows(q, H * d, "q"), k.data_ptr(), _rows(k, G * d, "k"), v.data_ptr(), _rows(v, G * e, "v"), _p(v_other), vos, float(lam),
-        q_start.data_ptr(), ctx_len.data_ptr(), seq_of_token.data_ptr(), _p(inv_freq), T, H, G, d, e, int(rot_dims), int(layout),
+        q_start.data_ptr(), ctx_len.data_ptr(), seq_of_token.data_ptr(), _p(inv_freq), float(mscale), T, H, G, d, e, int(rot_dims), int(layout),
         1 if qk_norm else 0, _p(q_weight), _p(k_weight), float(eps), _dt(q), _stream()), "rotary_qk_norm_kv_write")
     return q_out
 
@@ -927,3 +934,84 @@ def qk_row_norm_kv_write(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, k_ca
         k.data_ptr(), _rows(k, nk, "k"), v.data_ptr(), _rows(v, nv, "v"), q_weight.data_ptr(), k_weight.data_ptr(), T, nq, nk, nv,
         float(eps), _dt(q), _stream()), "qk_row_norm_kv_write")
     return q_out
+
+
+def conv_rotary_supported(dim: int, vdim: int, taps: int) -> bool:
+    """Head sizes and taps that ``conv_rotary_qk_norm_kv_write`` serves."""
+    return bool(_lib.mixers_lib().aphro_conv_rotary_supported(int(dim), int(vdim), int(taps)))
+
+
+def conv_rotary_qk_norm_kv_write(u: torch.Tensor, w: torch.Tensor, state: Optional[torch.Tensor], k_cache: torch.Tensor, v_cache: torch.Tensor,
+                                 slot_mapping: torch.Tensor, state_slots: torch.Tensor, q_start: torch.Tensor, q_len: torch.Tensor,
+                                 ctx_len: torch.Tensor, seq_of_token: torch.Tensor, max_q_len: int, heads: int, inv_freq: Optional[torch.Tensor],
+                                 rot_dims: int, mscale: float = 1.0, q_weight: Optional[torch.Tensor] = None,
+                                 k_weight: Optional[torch.Tensor] = None, eps: float = 1e-6) -> torch.Tensor:
+    """u [T, C]: the rows [q | k | v] of an input product (dense, any row stride), C = (heads + kv_heads) * dim + kv_heads * vdim.  Every
+    channel passes the short causal convolution w [C, taps] (state [slots, taps - 1, C], advanced), query and key heads are divided by
+    their root mean square times ``q_weight`` / ``k_weight`` [dim] (both None: no norm), the first ``rot_dims`` numbers of every query and
+    key head turn in pairs (i, i + rot_dims / 2), keys and values go into the paged caches, the queries [T, heads * dim] are returned.
+    ``max_q_len``: the batch's longest segment (host).  Sizes as ``conv_rotary_supported`` says."""
+    _cuda(u, w, state, k_cache, v_cache, slot_mapping, state_slots, q_start, q_len, ctx_len, seq_of_token, inv_freq, q_weight, k_weight)
+    nb, bs, G, d = k_cache.shape
+    e = v_cache.shape[3]
+    T, S = u.shape[0], q_start.numel()
+    C = (heads + G) * d + G * e
+    taps = w.shape[1]
+    _need(v_cache.shape[:3] == (nb, bs, G) and k_cache.is_contiguous() and v_cache.is_contiguous() and u.dtype == k_cache.dtype == v_cache.dtype,
+          "conv_rotary_qk_norm_kv_write: cache shapes / dtype")
+    _need(w.dim() == 2 and w.shape[0] == C and w.is_contiguous() and w.dtype == u.dtype, "conv_rotary_qk_norm_kv_write: w [channels, taps]")
+    _need(taps == 1 or (state is not None and state.dtype == u.dtype and state.dim() == 3 and state.is_contiguous()
+                        and tuple(state.shape[1:]) == (taps - 1, C)), "conv_rotary_qk_norm_kv_write: state [slots, taps - 1, channels]")
+    for t, nm in ((state_slots, "state_slots"), (q_start, "q_start"), (q_len, "q_len"), (ctx_len, "ctx_len")):
+        _i32(t, S, nm)
+    _i32(seq_of_token, T, "seq_of_token")
+    _need(slot_mapping.dtype == torch.int64 and slot_mapping.numel() == T and slot_mapping.is_contiguous(), "conv_rotary_qk_norm_kv_write: slots int64 [T]")
+    _need(rot_dims == 0 or (inv_freq is not None and inv_freq.dtype == torch.float32 and inv_freq.numel() == rot_dims // 2
+                            and inv_freq.is_contiguous()), "conv_rotary_qk_norm_kv_write: inv_freq fp32 [rot_dims / 2]")
+    _need((q_weight is None) == (k_weight is None), "conv_rotary_qk_norm_kv_write: a norm weight for queries and one for keys, or none")
+    for x in (q_weight, k_weight):
+        _need(x is None or (x.dtype == u.dtype and x.numel() == d and x.is_contiguous()), "conv_rotary_qk_norm_kv_write: norm weights [dim]")
+    q = torch.empty(T, heads * d, dtype=u.dtype, device=u.device)
+    check(_lib.mixers_lib().aphro_conv_rotary_qk_norm_kv_write(
+        q.data_ptr(), heads * d, k_cache.data_ptr(), v_cache.data_ptr(), slot_mapping.data_ptr(), nb * bs, u.data_ptr(),
+        _rows(u, C, "conv_rotary_qk_norm_kv_write u"), w.data_ptr(), _p(state) if taps > 1 else None, state_slots.data_ptr(), q_start.data_ptr(),
+        q_len.data_ptr(), ctx_len.data_ptr(), seq_of_token.data_ptr(), _p(inv_freq), float(mscale), _p(q_weight), _p(k_weight), float(eps), T, S,
+        int(max_q_len), heads, G, d, e, int(rot_dims), taps, _dt(u), _stream()), "conv_rotary_qk_norm_kv_write")
+    return q
+
+
+# ---- dynamic tanh around an fp32 residual ------------------------------------------------------------------------------------------
+def residual_tanh_norm(x: torch.Tensor, ya: Optional[torch.Tensor] = None, yb: Optional[torch.Tensor] = None,
+                       table: Optional[torch.Tensor] = None, ids: Optional[torch.Tensor] = None, norms=(), fresh: bool = False,
+                       dtype: Optional[torch.dtype] = None):
+    """x += ya + yb + table[ids] in place (fp32 [T, W]; every term optional; ``fresh``: x is written without being read), then one
+    tanh(alpha x) * w + b [T, W] in the activation dtype for every (alpha, w, b) of ``norms`` (up to two; alpha a host number)."""
+    T, W = x.shape
+    norms = list(norms)
+    _need(len(norms) <= 2, "residual_tanh_norm: up to two norms")
+    _cuda(x, ya, yb, table, ids, *[v for n in norms for v in n[1:]])
+    _need(x.dtype == torch.float32 and x.is_contiguous(), "residual_tanh_norm: x is fp32, contiguous")
+    some = next((t for t in [ya, yb, table] + [n[1] for n in norms] if t is not None), None)
+    adt = dtype or (some.dtype if some is not None else None)
+    _need(adt in _DT, "residual_tanh_norm: the activation dtype is not given")
+    st = []
+    for y in (ya, yb):
+        _need(y is None or (y.dtype == adt and y.shape[0] == T), "residual_tanh_norm: results [T, W] of the activation dtype")
+        st.append(0 if y is None else _rows(y, W, "residual_tanh_norm result"))
+    if table is not None:
+        _need(table.dtype == adt and table.dim() == 2 and table.shape[1] == W and table.is_contiguous() and ids is not None
+              and ids.dtype == torch.int64 and ids.numel() == T and ids.is_contiguous(), "residual_tanh_norm: table [vocab, W], ids int64 [T]")
+    args, outs = [], []
+    for i in range(2):
+        if i >= len(norms):
+            args += [0.0, None, None, None]
+            continue
+        alpha, w, b = norms[i]
+        for v in (w, b):
+            _need(v.dtype == adt and v.numel() == W and v.is_contiguous(), "residual_tanh_norm: weight and bias [W] of the activation dtype")
+        outs.append(torch.empty(T, W, dtype=adt, device=x.device))
+        args += [float(alpha), w.data_ptr(), b.data_ptr(), outs[-1].data_ptr()]
+    check(_lib.mixers_lib().aphro_residual_tanh_norm(x.data_ptr(), 1 if fresh else 0, _p(ya), st[0], _p(yb), st[1], _p(table),
+                                                     _p(ids) if table is not None else None, table.shape[0] if table is not None else 0, *args,
+                                                     T, W, _DT[adt], _stream()), "residual_tanh_norm")
+    return outs

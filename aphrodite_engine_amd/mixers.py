@@ -20,7 +20,7 @@ portions and decoded tokens in one launch -- through the kernels of ``mixer_ops`
                           token of every live request in a per-request slot
   RotaryFrequencies       rotation frequencies with YaRN's blend of interpolated and original frequencies and its magnitude factor
   LatentAttention         softmax attention through a low-rank latent: a token caches one row [normed latent | one rotated key part
-                          shared by all heads]; queries go through a latent of their own; elementwise sigmoid output gate
+                          shared by all heads]; queries go through a latent of their own; sigmoid output gate, elementwise or per head
   ClampedGLUMLP           down(g * sigmoid(alpha g) * (u + 1)) with g and u clamped, biased projections
   StreamedResidual        a residual carried as several streams that sublayers read through a learned combination and write back
                           through a learned mixing matrix (hyper-connections), with a per-channel scale on every sublayer's result
@@ -31,8 +31,12 @@ portions and decoded tokens in one launch -- through the kernels of ``mixer_ops`
                           keys and queries shared by groups of heads, behind a short convolution; gate, then RMS norm in parts
   GroupedQueryAttention   softmax attention of a fused input product's q, k and v rows: q / k normed per head before a (partial)
                           rotation or over the whole projection without one, masks / soft cap / distance bias / sink / gate as above
+                          and an optional short causal convolution on q, k and v ahead of all of it
   RotaryGQAttention       causal grouped-query softmax attention with a (partial) rotation, optional unit RMS of q and k after it
                           and optional blending of the values with an earlier layer's values of the same tokens
+  DynamicTanh             tanh(alpha x) w + b in the place of a norm: elementwise, no statistic
+  JoinedOutput            the output products of sublayers that run side by side as one product over their results
+  looped_layers           the order of layers of which a span runs several times in a row
 """
 import math
 from dataclasses import dataclass
@@ -192,17 +196,22 @@ class OuterProductMemory(nn.Module):
 
 
 class GatedMLP(nn.Module):
-    """down(act(gate x) * (up x)) with gate and up as one product."""
+    """down(act(gate x) * (up x)) with gate and up as one product.  ``down`` False: the output product is not this module's
+    (JoinedOutput); ``inner`` alone is used."""
 
-    def __init__(self, width: int, ff: int, act: int, dtype, prefix: str = ""):
+    def __init__(self, width: int, ff: int, act: int, dtype, prefix: str = "", down: bool = True):
         super().__init__()
         from .model import QuantLinear
-        self.act = act
+        self.act, self.ff = act, ff
         self.gate_up = QuantLinear(width, [ff, ff], None, dtype, prefix=prefix + "gate_up")
-        self.down = QuantLinear(ff, [width], None, dtype, prefix=prefix + "down")
+        self.down = QuantLinear(ff, [width], None, dtype, prefix=prefix + "down") if down else None
+
+    def inner(self, h: torch.Tensor, out: Optional[torch.Tensor] = None) -> torch.Tensor:
+        """What the output product reads, into ``out`` [T, ff] (dense rows, any row stride) if given."""
+        return mops.act_and_mul(self.gate_up(h), self.act, out)
 
     def forward(self, h: torch.Tensor) -> torch.Tensor:
-        return self.down(mops.act_and_mul(self.gate_up(h), self.act))
+        return self.down(self.inner(h))
 
 
 class WindowedMapsAttention(nn.Module):
@@ -431,11 +440,12 @@ class LatentAttention(nn.Module):
     returns sum_j p_ij c_j per head, and W_uv,a is applied to that, again batched over heads."""
 
     def __init__(self, width: int, heads: int, dim: int, rot_dim: int, vdim: int, q_rank: int, kv_rank: int, scale: float,
-                 rotary: RotaryFrequencies, eps: float, dtype, prefix: str = "", gate: bool = True, window: int = 0,
-                 sink: bool = False):
-        """``q_rank`` 0: queries are a plain projection of h (no query latent).  ``gate`` False: no output gate.  ``window`` > 0:
+                 rotary: RotaryFrequencies, eps: float, dtype, prefix: str = "", gate=True, window: int = 0,
+                 sink: bool = False, project: bool = True):
+        """``q_rank`` 0: queries are a plain projection of h (no query latent).  ``gate`` True: W_g has a row per output number, "head":
+        one per head (its sigmoid scales the head's output, in the attention's launch), False: no output gate.  ``window`` > 0:
         a row sees itself and the window - 1 tokens before it.  ``sink``: a learned number per head whose exponential joins the
-        softmax denominator."""
+        softmax denominator.  ``project`` False: W_o is not this module's (JoinedOutput); ``attend`` alone is used."""
         super().__init__()
         from .loader import merged_plan
         from .model import QuantLinear
@@ -443,9 +453,12 @@ class LatentAttention(nn.Module):
             raise ValueError(f"{rotary.dims} rotated numbers in a rotary part of {rot_dim}")
         self.heads, self.dim, self.rot_dim, self.vdim, self.q_rank, self.kv_rank = heads, dim, rot_dim, vdim, q_rank, kv_rank
         self.scale, self.eps, self.rotary = float(scale), float(eps), rotary
-        self.window, self.gated = max(int(window), 0), bool(gate)
+        if gate not in (True, False, "head"):
+            raise ValueError(f"output gate {gate!r}")
+        self.window, self.gated, self.head_gate = max(int(window), 0), bool(gate), gate == "head"
         self.names = ["dq" if q_rank else "q", "dkv"] + (["g"] if gate else [])
-        self.splits = [q_rank if q_rank else heads * (dim + rot_dim), kv_rank + rot_dim] + ([heads * vdim] if gate else [])
+        self.splits = [q_rank if q_rank else heads * (dim + rot_dim), kv_rank + rot_dim] + \
+            ([heads if self.head_gate else heads * vdim] if gate else [])
         self.n_named = len(self.splits)
         pad = -sum(self.splits) % 8               # rows of the fused product stay 16-byte multiples
         if pad:
@@ -457,8 +470,17 @@ class LatentAttention(nn.Module):
         self.uq = QuantLinear(q_rank, [heads * (dim + rot_dim)], None, dtype, prefix=prefix + "uq") if q_rank else None
         self.sink = nn.Parameter(torch.zeros(heads, dtype=torch.float32), requires_grad=False) if sink else None
         self.w_uk = nn.Parameter(torch.zeros(heads, dim, kv_rank, dtype=dtype), requires_grad=False)      # rows of W_uk, head by head
-        self.w_uv = nn.Parameter(torch.zeros(heads, vdim, kv_rank, dtype=dtype), requires_grad=False)
-        self.out_proj = QuantLinear(heads * vdim, [width], None, dtype, prefix=prefix + "out_proj")
+        self.w_uv = nn.Parameter(torch.zeros(heads, kv_rank, vdim, dtype=dtype), requires_grad=False)     # W_uv^T per head: a dense right operand
+        self.out_proj = QuantLinear(heads * vdim, [width], None, dtype, prefix=prefix + "out_proj") if project else None
+
+    def load_up_projection(self, key: str, t: torch.Tensor, name: str) -> None:
+        """W_uk ("uk", heads * dim rows) or W_uv ("uv", heads * vdim rows), laid out head by head in the checkpoint."""
+        n = self.dim if key == "uk" else self.vdim
+        if tuple(t.shape) != (self.heads * n, self.kv_rank):
+            raise ValueError(f"{name}: checkpoint tensor {tuple(t.shape)} does not fit {(self.heads * n, self.kv_rank)}")
+        t = t.reshape(self.heads, n, self.kv_rank)
+        dst = self.w_uk if key == "uk" else self.w_uv
+        dst.data.copy_((t if key == "uk" else t.transpose(1, 2)).to(dst.dtype))
 
     def cache_spec(self) -> LatentCacheSpec:
         return LatentCacheSpec(self.kv_rank, self.rot_dim)
@@ -466,7 +488,9 @@ class LatentAttention(nn.Module):
     def finalize(self) -> None:
         self.rotary.to(self.w_uk.device)
 
-    def forward(self, h: torch.Tensor, cache: torch.Tensor, batch: StepBatch) -> torch.Tensor:
+    def attend(self, h: torch.Tensor, cache: torch.Tensor, batch: StepBatch, out: Optional[torch.Tensor] = None,
+               rows: Optional[torch.Tensor] = None) -> torch.Tensor:
+        """The gated heads [T, heads * vdim], into ``out`` (dense rows, any row stride) if given; ``rows``: of these rows only."""
         T, H, d, P, e, R = h.shape[0], self.heads, self.dim, self.rot_dim, self.vdim, self.kv_rank
         rot = self.rotary
         proj = self.in_proj(h)
@@ -476,20 +500,27 @@ class LatentAttention(nn.Module):
             q = self.uq(cq).view(T, H, d + P)
         else:
             q = proj.as_strided((T, H, d + P), (proj.stride(0), d + P, 1))
+        g_at = self.splits[0] + R + P
         q_lat = torch.empty(T, H, R, dtype=h.dtype, device=h.device)
         torch.bmm(q[:, :, :d].transpose(0, 1), self.w_uk, out=q_lat.transpose(0, 1))
         o_lat = torch.empty(T, H, R, dtype=h.dtype, device=h.device)
         mops.latent_attention(o_lat, q_lat, q[:, :, d:] if P else None, cache, batch.block_tables, batch.q_start, batch.q_len,
                               batch.ctx_len, batch.seq_of_token, (min(batch.q_lens), max(batch.q_lens)), rot.inv_freq, rot.mscale,
                               rot.dims, self.scale, max_kv_len=max(c + n for c, n in zip(batch.ctx_lens, batch.q_lens)),
-                              window=self.window, sink=self.sink)
-        o = torch.empty(T, H, e, dtype=h.dtype, device=h.device)
-        torch.bmm(o_lat.transpose(0, 1), self.w_uv.transpose(1, 2), out=o.transpose(0, 1))
-        o = o.view(T, H * e)
-        if self.gated:
-            g_at = self.splits[0] + R + P
-            mops.sigmoid_gate_mul(o, proj[:, g_at:g_at + H * e], out=o)
-        return self.out_proj(o)
+                              window=self.window, sink=self.sink, gate=proj[:, g_at:g_at + H] if self.head_gate else None)
+        if rows is not None:
+            o_lat = o_lat.index_select(0, rows)
+        n = o_lat.shape[0]
+        if out is None:
+            out = torch.empty(n, H * e, dtype=h.dtype, device=h.device)
+        torch.bmm(o_lat.transpose(0, 1), self.w_uv, out=out.as_strided((H, n, e), (e, out.stride(0), 1)))
+        if self.gated and not self.head_gate:
+            gate = proj[:, g_at:g_at + H * e]
+            mops.sigmoid_gate_mul(out, gate if rows is None else gate.index_select(0, rows), out=out)
+        return out
+
+    def forward(self, h: torch.Tensor, cache: torch.Tensor, batch: StepBatch) -> torch.Tensor:
+        return self.out_proj(self.attend(h, cache, batch))
 
 
 class ClampedGLUMLP(nn.Module):
@@ -641,10 +672,12 @@ class GroupedQueryAttention(nn.Module):
     product (and the raw rows of an elementwise sigmoid gate) and leaves the heads' outputs.  ``qk_norm``: None, "head" (RMS norm of
     every head with a weight shared by the heads, before the rotation) or "row" (RMS norm over the whole projection; no rotation).
     ``rotary`` turns the first ``rotary.dims`` numbers of every head in the given pair ``layout``.  Masks, soft cap, distance bias and
-    sink are DistanceBiasAttention's, whose kernels it runs."""
+    sink are DistanceBiasAttention's, whose kernels it runs.  ``taps`` > 0: every channel of q, k and v first passes a short causal
+    convolution over time (its last inputs live in a per-request slot); convolution, norm, rotation and cache write are one launch
+    where the sizes allow it."""
 
     def __init__(self, heads: int, kv_heads: int, dim: int, vdim: int, scale: float, eps: float, dtype, qk_norm: Optional[str] = None,
-                 rotary: Optional[RotaryFrequencies] = None, layout: int = mops.ROTARY_HALF, **attention):
+                 rotary: Optional[RotaryFrequencies] = None, layout: int = mops.ROTARY_HALF, taps: int = 0, **attention):
         super().__init__()
         if qk_norm not in (None, "head", "row"):
             raise ValueError(f"qk_norm {qk_norm!r}")
@@ -660,9 +693,14 @@ class GroupedQueryAttention(nn.Module):
         nq, nk = (heads * dim, kv_heads * dim) if qk_norm == "row" else (dim, dim)
         self.q_norm = nn.Parameter(torch.ones(nq, dtype=dtype), requires_grad=False) if qk_norm else None
         self.k_norm = nn.Parameter(torch.ones(nk, dtype=dtype), requires_grad=False) if qk_norm else None
+        self.taps, self.channels = int(taps), sum(self.splits)
+        self.conv = nn.Parameter(torch.zeros(self.channels, self.taps, dtype=dtype), requires_grad=False) if taps else None
 
     def cache_spec(self) -> PagedKVSpec:
         return self.attn.cache_spec()
+
+    def state_spec(self) -> ConvStateSpec:
+        return ConvStateSpec(self.channels, self.taps)
 
     def finalize(self, device) -> None:
         self.rotary.to(device)
@@ -676,8 +714,24 @@ class GroupedQueryAttention(nn.Module):
         else:
             q = mops.rotary_qk_norm_kv_write(q, k, v, k_cache, v_cache, batch.slot_mapping, batch.q_start, batch.ctx_len,
                                              batch.seq_of_token, self.rotary.inv_freq, self.rotary.dims, self.layout,
-                                             self.qk_norm is not None, self.eps, q_weight=self.q_norm, k_weight=self.k_norm)
+                                             self.qk_norm is not None, self.eps, q_weight=self.q_norm, k_weight=self.k_norm,
+                                             mscale=self.rotary.mscale)
         self.attn.attend(out, q, gate, cache, batch, out_scale)
+
+    def forward_conv(self, out: torch.Tensor, qkv: torch.Tensor, gate: Optional[torch.Tensor], cache, conv_state: Optional[torch.Tensor],
+                     batch: StepBatch, out_scale: float = 1.0) -> None:
+        """``forward`` with the convolution in front: qkv [T, channels] are the rows [q | k | v] of an input product."""
+        k_cache, v_cache = cache
+        if self.layout == mops.ROTARY_HALF and self.qk_norm != "row" and qkv.stride(0) % 8 == 0 \
+                and mops.conv_rotary_supported(self.dim, self.vdim, self.taps):
+            q = mops.conv_rotary_qk_norm_kv_write(qkv, self.conv, conv_state, k_cache, v_cache, batch.slot_mapping, batch.state_slots,
+                                                  batch.q_start, batch.q_len, batch.ctx_len, batch.seq_of_token, max(batch.q_lens), self.heads,
+                                                  self.rotary.inv_freq, self.rotary.dims, self.rotary.mscale, self.q_norm, self.k_norm, self.eps)
+            self.attn.attend(out, q, gate, cache, batch, out_scale)
+            return
+        u = mops.short_conv(qkv, self.conv, conv_state, batch.state_slots, batch.q_start, batch.q_len, batch.ctx_len, batch.seq_of_token,
+                            self.channels)
+        self.forward(out, *u.split(self.splits, dim=1), gate, cache, batch, out_scale)
 
 
 class RotaryGQAttention(nn.Module):
@@ -728,3 +782,66 @@ class RotaryGQAttention(nn.Module):
                                      batch.seq_of_token, (min(batch.q_lens), max(batch.q_lens)), H, self.scale, None,
                                      max_kv_len=max(c + n for c, n in zip(batch.ctx_lens, batch.q_lens)))
         return self.out_proj(o), v
+
+
+class DynamicTanh(nn.Module):
+    """tanh(alpha x) w + b with a learned scalar alpha: stands where a norm would.  ``operand`` is what ``residual_tanh_norm`` takes."""
+
+    def __init__(self, width: int, dtype):
+        super().__init__()
+        self.weight = nn.Parameter(torch.ones(width, dtype=dtype), requires_grad=False)
+        self.bias = nn.Parameter(torch.zeros(width, dtype=dtype), requires_grad=False)
+        self.alpha = nn.Parameter(torch.ones((), dtype=torch.float32), requires_grad=False)
+        self.alpha_value = 1.0
+
+    def finalize(self) -> None:
+        self.alpha_value = float(self.alpha)
+
+    def operand(self) -> Tuple[float, torch.Tensor, torch.Tensor]:
+        return self.alpha_value, self.weight, self.bias
+
+
+class JoinedOutput(nn.Module):
+    """sum_i W_i y_i of sublayers that run side by side, as ONE product: their results y_i stand next to one another in the rows of a
+    buffer (each from a multiple of 8 on, so that every piece can be written 16 bytes at a time) and so do the W_i."""
+
+    def __init__(self, sizes: List[int], width: int, dtype, prefix: str = ""):
+        super().__init__()
+        from .model import QuantLinear
+        self.sizes, self.at, a = list(sizes), [], 0
+        for n in self.sizes:
+            self.at.append(a)
+            a += (n + 7) // 8 * 8
+        self.padded = a != sum(self.sizes)
+        self.total = a
+        self.linear = QuantLinear(a, [width], None, dtype, prefix=prefix)
+        self.linear.weight.data.zero_()
+
+    def weight_of(self, i: int) -> torch.Tensor:
+        return self.linear.weight.data[:, self.at[i]:self.at[i] + self.sizes[i]]
+
+    def zero_padding(self) -> None:
+        """After random filling: the columns between the pieces are zero."""
+        for i, n in enumerate(self.sizes):
+            end = self.at[i + 1] if i + 1 < len(self.at) else self.total
+            self.linear.weight.data[:, self.at[i] + n:end].zero_()
+
+    def buffer(self, rows: int, dtype, device) -> Tuple[torch.Tensor, List[torch.Tensor]]:
+        """([rows, total], its pieces as views); the columns between the pieces are zero."""
+        make = torch.zeros if self.padded else torch.empty
+        buf = make(rows, self.total, dtype=dtype, device=device)
+        return buf, [buf[:, a:a + n] for a, n in zip(self.at, self.sizes)]
+
+    def forward(self, buf: torch.Tensor) -> torch.Tensor:
+        return self.linear(buf)
+
+
+def looped_layers(count: int, start: int = 0, stop: int = 0, times: int = 1) -> List[Tuple[int, bool]]:
+    """The order in which ``count`` layers run when layers start .. stop - 1 run ``times`` times in a row: (layer, whether a further
+    pass over the span begins with it)."""
+    if not (0 <= start <= stop <= count and times >= 1):
+        raise ValueError(f"layers {start} .. {stop} of {count}, {times} times")
+    runs = [(i, False) for i in range(start)]
+    for n in range(times):
+        runs += [(i, n > 0 and i == start) for i in range(start, stop)]
+    return runs + [(i, False) for i in range(stop, count)]

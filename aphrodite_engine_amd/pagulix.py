@@ -324,10 +324,8 @@ class PagulixForCausalLM(nn.Module):
                 return put(mix.kv_norm.data, t, name)
             elif key == "sink":
                 return put(mix.sink.data, t, name)
-            elif key == "uk":
-                return put(mix.w_uk.data.view(mix.heads * mix.dim, mix.kv_rank), t, name)
-            elif key == "uv":
-                return put(mix.w_uv.data.view(mix.heads * mix.vdim, mix.kv_rank), t, name)
+            elif key in ("uk", "uv"):
+                return mix.load_up_projection(key, t, name)
         elif key == "vmix":
             return None if mix.v_blend is None else put(mix.v_blend.data, t.reshape(()), name)
         lin = mix.in_proj

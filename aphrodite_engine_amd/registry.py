@@ -68,6 +68,10 @@ def _register_builtin() -> None:
         from .nukezen import load_nukezen
         return load_nukezen(model_dir, config, **kw)
 
+    def vivisun(model_dir, config, **kw):
+        from .vivisun import load_vivisun
+        return load_vivisun(model_dir, config, **kw)
+
     for arch in ("LlamaForCausalLM", "MistralForCausalLM", "MixtralForCausalLM"):
         _LOADERS.setdefault(arch, llama)
     _LOADERS.setdefault("Fatudra", fatudra)
@@ -75,3 +79,4 @@ def _register_builtin() -> None:
     _LOADERS.setdefault("Fekotar", fekotar)
     _LOADERS.setdefault("Pagulix", pagulix)
     _LOADERS.setdefault("Nukezen", nukezen)
+    _LOADERS.setdefault("Vivisun", vivisun)

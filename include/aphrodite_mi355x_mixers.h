@@ -59,8 +59,8 @@ int aphro_silu_gate_part_rms_norm(void* out, int64_t out_stride, const float* x,
                                   void* stream);
 
 /* out[t, j] = act(in[t, j]) * in[t, d + j], j < d.  act: 0 silu, 1 gelu (tanh form).  in [T, 2 d] (row stride in_stride),
- * out [T, d] contiguous; math in fp32, one rounding. */
-int aphro_act_and_mul(void* out, const void* in, int64_t in_stride, int64_t num_tokens, int d, int act, int dtype,
+ * out [T, d] (row stride out_stride); math in fp32, one rounding. */
+int aphro_act_and_mul(void* out, int64_t out_stride, const void* in, int64_t in_stride, int64_t num_tokens, int d, int act, int dtype,
                       void* stream);
 
 /* out[t, n] = out_scale * x[t, n] / rms(group of n) * weight[n] * sigmoid(gate[t, n]);  x fp32 [T, N] contiguous, groups of
@@ -145,6 +145,10 @@ int aphro_poly_norm(void* out, const void* z, int64_t z_stride, int64_t num_toke
 int aphro_differential_norm_gate(void* out, int64_t out_stride, const float* a, int64_t a_stride, const void* gate,
                                  int64_t gate_stride, int64_t num_tokens, int heads, int maps, int vdim, float lambda,
                                  float out_scale, float eps, int dtype, void* stream);
+
+/* The second half of aphro_short_conv alone: every segment's slot takes the last taps - 1 inputs u of its sequence. */
+int aphro_short_conv_state(void* state, const void* u, int64_t u_stride, const int32_t* state_slots, const int32_t* q_start,
+                           const int32_t* q_len, const int32_t* ctx_len, int num_seqs, int channels, int taps, int dtype, void* stream);
 
 /* Short causal convolution over time on each channel of u [T, cq + ck + cv] (row stride u_stride):
  *   y_t[c] = sum_j w[c, j] * u_(t - taps + 1 + j)[c] + bias[c],  zeros before the sequence's start;  w [channels, taps] and
@@ -242,6 +246,13 @@ int aphro_token_state_write(int32_t* token_state, const int64_t* ids, const int3
 int aphro_residual_add2_rms_norm(float* x, const void* ya, int64_t ya_stride, const void* yb, int64_t yb_stride, const void* bias,
                                  const void* weight, void* out, int64_t num_tokens, int width, float eps, int dtype, void* stream);
 
+/* Around an fp32 residual stream whose norms are dynamic tanhs, norm(r) = tanh(alpha r) * w + b:
+ *   x += ya + yb + table[ids[t]]   (each optional; fresh != 0: x is written, not read),  out1 = norm1(x), out2 = norm2(x) (NULL: not)
+ * x fp32 [T, width]; ya, yb (row strides), table [vocab, width], w, b [width] and out [T, width] (contiguous) of `dtype`. */
+int aphro_residual_tanh_norm(float* x, int fresh, const void* ya, int64_t ya_stride, const void* yb, int64_t yb_stride, const void* table,
+                             const int64_t* ids, int64_t vocab, float alpha1, const void* w1, const void* b1, void* out1, float alpha2,
+                             const void* w2, const void* b2, void* out2, int64_t num_tokens, int width, int dtype, void* stream);
+
 /* Per token, from the rows of one input product (proj, row stride proj_stride): cq[t] = rms_norm(proj[t, q_at : q_at + q_rank]) *
  * wq (q_rank 0: none); cache[slot_mapping[t]] = [rms_norm(proj[t, kv_at : kv_at + kv_rank]) * wkv | rotate(next rot_dim numbers)].
  * cache [num_cache_rows, kv_rank + rot_dim].  The rotation turns pair (i, i + rot_dims / 2) of the first rot_dims numbers by
@@ -254,15 +265,16 @@ int aphro_latent_prep(void* cq, void* cache, int64_t num_cache_rows, const void*
  * score = ([q_lat | rotate(q_rot)] . row) * scale, out = sum p * row[:kv_rank].  q_lat / q_rot / out are addressed as
  * base + t * stride + head * head_stride (elements); any sizes (kv_rank <= 1024), fp32 math.
  * window > 0: row i sees key j only if i - j < window.  sink fp32 [heads] (NULL: none): exp(sink[head]) -- not scaled -- is
- * one more term of the softmax denominator, without a value. */
+ * one more term of the softmax denominator, without a value.  gate [T, heads] of `dtype` (row stride; NULL: none): a head's output is
+ * multiplied by sigmoid(gate[t, head]). */
 int aphro_latent_attention_plain(void* out, int64_t out_stride, int64_t out_head_stride, const void* q_lat, int64_t ql_stride,
                                  int64_t ql_head_stride, const void* q_rot, int64_t qr_stride, int64_t qr_head_stride,
                                  const void* cache, const int32_t* block_tables, int max_blocks, int64_t num_blocks, int block_size,
                                  const int32_t* q_start, const int32_t* ctx_len, const int32_t* seq_of_token, const float* inv_freq,
                                  float mscale, int64_t num_tokens, int heads, int kv_rank, int rot_dim, int rot_dims, float scale,
-                                 int window, const float* sink, int dtype, void* stream);
+                                 int window, const float* sink, const void* gate, int64_t gate_stride, int dtype, void* stream);
 /* The same attention with the kernel chosen by size: bf16 with (kv_rank, rot_dim) in {(128, 16), (128, 32), (256, 32), (256, 64),
- * (512, 64)}, rot_dims == rot_dim and 16-byte aligned rows run on the matrix cores (aphro_latent_attention_fast_supported), the
+ * (512, 64)} or, without a rotary part, kv_rank in {64, 96, 128, 192, 256, 384, 512}, rot_dims == rot_dim and 16-byte aligned rows run on the matrix cores (aphro_latent_attention_fast_supported), the
  * query rows of a segment flattened to (token, head) pairs, 64 per workgroup; everything else runs the kernel above.  min/max
  * segment lengths and the longest ctx_len + q_len come from the host.  Decode-sized launches split long key ranges over
  * aphro_latent_attention_splits(...) workgroups when `workspace` holds num_tokens * heads * splits * (2 + kv_rank) floats. */
@@ -273,8 +285,8 @@ int aphro_latent_attention(void* out, int64_t out_stride, int64_t out_head_strid
                            const int32_t* block_tables, int max_blocks, int64_t num_blocks, int block_size, const int32_t* q_start,
                            const int32_t* q_len, const int32_t* ctx_len, const int32_t* seq_of_token, const float* inv_freq,
                            float mscale, int64_t num_tokens, int num_seqs, int max_q_len, int max_kv_len, int heads, int kv_rank,
-                           int rot_dim, int rot_dims, float scale, int window, const float* sink, float* workspace,
-                           int64_t workspace_floats, int dtype, void* stream);
+                           int rot_dim, int rot_dims, float scale, int window, const float* sink, const void* gate, int64_t gate_stride,
+                           float* workspace, int64_t workspace_floats, int dtype, void* stream);
 /* out[t, i] = x[t, i] * sigmoid(gate[t, i]), i < n (out may be x) */
 int aphro_sigmoid_gate_mul(void* out, int64_t out_stride, const void* x, int64_t x_stride, const void* gate, int64_t gate_stride,
                            int64_t num_tokens, int n, int dtype, void* stream);
@@ -324,7 +336,7 @@ int aphro_gated_head_rms_norm(void* out, int64_t out_stride, const float* x, con
                               void* stream);
 
 /* From the rows of a rotary attention's input product: the first rot_dims numbers of every query and key head turned by
- * position * inv_freq[i] (layout 0: number i pairs with i + rot_dims / 2; 1: number 2 i with 2 i + 1), then -- qk_norm != 0 --
+ * position * inv_freq[i] (layout 0: number i pairs with i + rot_dims / 2; 1: number 2 i with 2 i + 1; cos and sin times mscale), then -- qk_norm != 0 --
  * every query and key head divided by sqrt(mean(x^2) + eps), times -- before the rotation -- q_weight [dim] or k_weight [dim] of
  * `dtype`, shared by the heads (NULL: none); values blended v <- (1 - lambda) v + lambda v_other (v_other NULL:
  * none).  Queries go to q_out [T, heads * dim], keys and values into k_cache [rows, kv_heads, dim] / v_cache [rows, kv_heads,
@@ -333,8 +345,22 @@ int aphro_rotary_qk_norm_kv_write(void* q_out, int64_t q_out_stride, void* k_cac
                                   int64_t num_cache_rows, const void* q, int64_t q_stride, const void* k, int64_t k_stride,
                                   const void* v, int64_t v_stride, const void* v_other, int64_t v_other_stride, float lambda,
                                   const int32_t* q_start, const int32_t* ctx_len, const int32_t* seq_of_token, const float* inv_freq,
-                                  int64_t num_tokens, int heads, int kv_heads, int dim, int vdim, int rot_dims, int layout,
+                                  float mscale, int64_t num_tokens, int heads, int kv_heads, int dim, int vdim, int rot_dims, int layout,
                                   int qk_norm, const void* q_weight, const void* k_weight, float eps, int dtype, void* stream);
+
+/* The preparation of a rotary attention whose q, k and v pass a short causal convolution over time, in one launch.  u [T, C] (row
+ * stride), C = (heads + kv_heads) * dim + kv_heads * vdim channels [q | k | v]; w [C, taps] and state [slots, taps - 1, C] as in
+ * aphro_short_conv (the state is advanced); then query and key heads divided by sqrt(mean(x^2) + eps) and times q_weight / k_weight
+ * [dim] (NULL, both: no norm), then the rotation of the first rot_dims numbers (pairs i, i + rot_dims / 2; cos and sin times mscale);
+ * queries go to q_out, keys and values into the paged caches at slot_mapping[t].  dim and vdim multiples of 8 (<= 512), taps 1 .. 4
+ * (aphro_conv_rotary_supported), every row 16-byte aligned.  max_q_len: the longest segment (1: the states advance in the same launch). */
+int aphro_conv_rotary_supported(int dim, int vdim, int taps);
+int aphro_conv_rotary_qk_norm_kv_write(void* q_out, int64_t q_out_stride, void* k_cache, void* v_cache, const int64_t* slot_mapping,
+                                       int64_t num_cache_rows, const void* u, int64_t u_stride, const void* w, void* state,
+                                       const int32_t* state_slots, const int32_t* q_start, const int32_t* q_len, const int32_t* ctx_len,
+                                       const int32_t* seq_of_token, const float* inv_freq, float mscale, const void* q_weight,
+                                       const void* k_weight, float eps, int64_t num_tokens, int num_seqs, int max_q_len, int heads,
+                                       int kv_heads, int dim, int vdim, int rot_dims, int taps, int dtype, void* stream);
 
 /* An attention's preparation without rotation: q [T, nq] and k [T, nk] (row strides), every row at once divided by
  * sqrt(mean(row^2) + eps) and times q_weight [nq] / k_weight [nk]; queries go to q_out [T, nq], keys and the values v [T, nv] as

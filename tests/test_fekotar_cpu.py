@@ -65,7 +65,7 @@ def test_loader_fills_fused_products_and_refuses_wrong_checkpoints(tmp_path):
     np.testing.assert_array_equal(w[112:112 + 120], W["l0.mix.g"])
     assert w.shape[0] % 8 == 0 and not w[232:].any()
     np.testing.assert_array_equal(mix.w_uk.detach().numpy().reshape(3 * 24, 48), W["l0.mix.uk"])
-    np.testing.assert_array_equal(mix.w_uv.detach().numpy().reshape(3 * 40, 48), W["l0.mix.uv"])
+    np.testing.assert_array_equal(mix.w_uv.detach().numpy().transpose(0, 2, 1).reshape(3 * 40, 48), W["l0.mix.uv"])
     np.testing.assert_array_equal(mix.q_norm.detach().numpy(), W["l0.mix.dq.norm"])
     mlp = m.layers[0].mlp
     np.testing.assert_array_equal(mlp.gate_up.weight.detach().numpy(), np.concatenate([W["l0.mlp.gate"], W["l0.mlp.up"]]))

@@ -1,4 +1,4 @@
-"""``bench.py --mixers [--mixers-design fatudra|gipozen|fekotar|pagulix|nukezen]``: prefill and decode throughput of a Fatudra (or Gipozen) stack at sizes that resemble a real model's layers
+"""``bench.py --mixers [--mixers-design fatudra|gipozen|fekotar|pagulix|nukezen|vivisun]``: prefill and decode throughput of a Fatudra (or Gipozen) stack at sizes that resemble a real model's layers
 (random bf16 weights), beside a Llama stack of equal width / heads / feed-forward / layer count on the unquantised op path,
 plus each mixer kernel alone against its roofline and against the like kernel of the Llama path.  Prints ONE JSON line;
 the default workload of bench.py is untouched by it.  The Gipozen stack: windowed differential attention (two maps of half the
@@ -21,6 +21,11 @@ The Nukezen stack: a channel-delta layer (16 / 32 heads of 128 x 128 state, inne
 tensors, and a chunked attention layer (chunks of 2048, soft cap, distance bias, sink), a dense gelu feed-forward in every layer; it
 stands beside the Fatudra stack (the closest existing model: attention beside a memory, post-norms, the same feed-forward), the
 Pagulix stack (the other delta rule) and Llama.
+
+The Vivisun stack: two layers -- rotary attention (half of every head rotates, 4-tap convolutions, elementwise gate) and a latent
+attention of rank 512 without a rotated part (sinks, a gate per head) -- that run twice in a row (four layer runs), a dense silu
+feed-forward beside every mixer; it stands beside the Fekotar stack (the closest existing model: sublayers side by side, attention
+through a latent) and Llama.
 
 Rooflines used: 8 TB/s HBM for the memory-bound kernels (norms, activations, decode attention, the decode step of the
 memories: their state is read and written once), 2.5 PFLOP/s dense bf16 MFMA for prompt attention (4 d flops per visible
@@ -821,8 +826,167 @@ def main_nukezen(args) -> int:
     return 0
 
 
+VIV_RANK, VIV_TAPS, VIV_PASSES = 512, 4, 2
+
+
+def vivisun_config(s):
+    """attention, latent attention, run twice in a row: four layer runs on two layers' weights."""
+    H, G, d = s["heads"], s["kv_heads"], s["dim"]
+    dense = {"kind": "dense", "ff": s["ff"]}
+    attn = {"type": "attention", "mlp": dense,
+            "mixer": {"heads": H, "kv_heads": G, "dim": d, "vdim": d, "conv": VIV_TAPS, "scale": d ** -0.5,
+                      "rot": {"base": 10000.0, "dims": d // 2, "scaling": {"factor": 4.0, "original": 4096, "fast": 32.0, "slow": 1.0}}}}
+    latent = {"type": "latent_attention", "mlp": dense,
+              "mixer": {"heads": H, "dim": d, "vdim": d, "kv_rank": VIV_RANK, "scale": d ** -0.5}}
+    return {"architecture": "Vivisun", "vocab": VOCAB, "width": s["width"], "norm": {"eps": 1e-6}, "layers": [attn, latent],
+            "loop": {"start": 0, "stop": 2, "times": VIV_PASSES}}
+
+
+def vivisun_kernel_section(s, prompt_len, batch, ctx, device):
+    """Each kernel that Vivisun adds (or extends) alone at the stack's shapes, beside the like kernel of the closest existing path."""
+    from . import mixer_ops as mops
+    from .mixers import LatentCacheSpec, RotaryFrequencies
+    bf = torch.bfloat16
+    H, G, d, W, ff, R, P = s["heads"], s["kv_heads"], s["dim"], s["width"], s["ff"], VIV_RANK, FEK_ROT
+    pre, dec, pages = batches(prompt_len, batch, ctx, device, VOCAB)
+    out = {}
+
+    def rec(name, sec, like, lsec, bytes_=None, flops=None, lbytes=None, lflops=None):
+        """lbytes / lflops: the like kernel's work where it differs."""
+        r, lr = {"us": round(sec * 1e6, 1)}, {"kernel": like, "us": round(lsec * 1e6, 1)}
+        if bytes_ is not None:
+            r["frac_hbm"], lr["frac_hbm"] = round(bytes_ / sec / HBM, 3), round((lbytes or bytes_) / lsec / HBM, 3)
+        if flops is not None:
+            r["frac_mfma"], lr["frac_mfma"] = round(flops / sec / MFMA, 4), round((lflops or flops) / lsec / MFMA, 4)
+        r["like"] = lr
+        out[name] = r
+
+    rn = lambda *shape, dtype=bf: torch.randn(*shape, device=device, dtype=dtype)
+    rot = RotaryFrequencies(d // 2, 10000.0, 4.0, 4096, 32.0, 1.0).to(device)
+    rotP = RotaryFrequencies(P, 10000.0, 4.0, 4096, 32.0, 1.0).to(device)
+    kc, vc = rn(pages, BLOCK, G, d), rn(pages, BLOCK, G, d)
+    cache, cacheP = (LatentCacheSpec(R, p).allocate(pages, BLOCK, batch, bf, device).normal_() for p in (0, P))
+    table, pair = rn(VOCAB, W), rn(65522, W)
+    C = (H + 2 * G) * d
+    for name, b, T in (("prefill", pre, prompt_len), ("decode", dec, batch)):
+        seg = (b.state_slots, b.q_start, b.q_len, b.ctx_len)
+        lens = (min(b.q_lens), max(b.q_lens))
+        kvmax = max(c + q for c, q in zip(b.ctx_lens, b.q_lens))
+        # ---- the launch between the layers, the embedding's -----------------------------------------------------------------------
+        x, ya, yb, w16, b16 = rn(T, W, dtype=torch.float32), rn(T, W), rn(T, W), rn(W), rn(W)
+        two = [(0.5, w16, b16), (0.7, w16, b16)]
+        lsec = timed(lambda: mops.residual_add2_rms_norm(x, ya, yb, weight=w16))
+        x.normal_()
+        sec = timed(lambda: mops.residual_tanh_norm(x, ya, norms=two))
+        rec("residual_tanh_norm_" + name, sec, "residual_add2_rms_norm", lsec, bytes_=T * W * 14)
+        sec = timed(lambda: mops.residual_tanh_norm(x, ya, table=table, ids=b.input_ids, norms=two))
+        rec("residual_tanh_norm_with_embedding_" + name, sec, "residual_add2_rms_norm", lsec, bytes_=T * W * 16, lbytes=T * W * 14)
+        tstate = torch.zeros(batch, dtype=torch.int32, device=device)
+        sec = timed(lambda: mops.residual_tanh_norm(x, table=table, ids=b.input_ids, norms=two, fresh=True))
+        lsec = timed(lambda: mops.hashed_pair_embed(table, pair, b.input_ids, tstate, *seg, b.seq_of_token, 131, 3))
+        rec("embed_tanh_norm_" + name, sec, "hashed_pair_embed", lsec, bytes_=T * W * 10, lbytes=T * W * 8)
+        # ---- preparation of the rotary attention: one launch beside two ---------------------------------------------------------------
+        proj = rn(T, C + H * d)
+        u, g = proj[:, :C], proj[:, C:]
+        cw, wh = rn(C, VIV_TAPS), rn(d)
+        state = torch.zeros(batch, VIV_TAPS - 1, C, device=device, dtype=bf)
+        sec = timed(lambda: mops.conv_rotary_qk_norm_kv_write(u, cw, state, kc, vc, b.slot_mapping, *seg, b.seq_of_token, lens[1], H, rot.inv_freq,
+                                                              d // 2, rot.mscale, wh, wh, 1e-6))
+
+        def apart():
+            y = mops.short_conv(u, cw, state, *seg, b.seq_of_token, C)
+            mops.rotary_qk_norm_kv_write(y[:, :H * d], y[:, H * d:(H + G) * d], y[:, (H + G) * d:], kc, vc, b.slot_mapping, b.q_start, b.ctx_len,
+                                         b.seq_of_token, rot.inv_freq, d // 2, mops.ROTARY_HALF, True, 1e-6, q_weight=wh, k_weight=wh, mscale=rot.mscale)
+        lsec = timed(apart)
+        rec("conv_rotary_qk_norm_kv_write_" + name, sec, "short_conv, then rotary_qk_norm_kv_write", lsec, bytes_=T * C * 4, lbytes=T * C * 8)
+        # ---- the rotary attention with its elementwise gate ---------------------------------------------------------------------------
+        q, o = rn(T, H * d), torch.empty(T, H * d, device=device, dtype=bf)
+        run = lambda gate: mops.distance_bias_attention(o, q, gate, kc, vc, b.block_tables, b.q_start, b.q_len, b.ctx_len, b.seq_of_token, lens, H,
+                                                        d ** -0.5, None, max_kv_len=kvmax)
+        kc.normal_()
+        vc.normal_()
+        sec, lsec = timed(lambda: run(g)), timed(lambda: run(None))
+        pairs = T * (T + 1) / 2
+        if name == "prefill":
+            rec("attention_prefill", sec, "the same launch, no gate", lsec, flops=pairs * H * 4.0 * d)
+        else:
+            rec("attention_decode", sec, "the same launch, no gate", lsec, bytes_=batch * (ctx + 1) * G * 2 * d * 2)
+        # ---- the latent attention: no rotated part, sinks, a gate per head -------------------------------------------------------------
+        q_lat, hg, sink = rn(T, H, R) * R ** -0.5, rn(T, H), torch.zeros(H, device=device)
+        qP, ol = rn(T, H, P), torch.empty(T, H, R, device=device, dtype=bf)
+        lat = lambda c, qr, r, dims, **kw: mops.latent_attention(ol, q_lat, qr, c, b.block_tables, b.q_start, b.q_len, b.ctx_len, b.seq_of_token, lens,
+                                                                 r.inv_freq, r.mscale, dims, d ** -0.5, max_kv_len=kvmax, **kw)
+        sec = timed(lambda: lat(cache, None, rot, 0, sink=sink, gate=hg))
+        lsec = timed(lambda: lat(cacheP, qP, rotP, P))
+        if name == "prefill":
+            rec("latent_attention_prefill", sec, "latent_attention with a rotated part of 64", lsec, flops=pairs * H * 4.0 * R,
+                lflops=pairs * H * (4.0 * R + 2.0 * P))
+        else:
+            rec("latent_attention_decode", sec, "latent_attention with a rotated part of 64", lsec, bytes_=batch * (ctx + 1) * R * 2,
+                lbytes=batch * (ctx + 1) * (R + P) * 2)
+        lp = rn(T, H * d + R + P)
+        wkv = rn(R)
+        prep = lambda c, p, r, dims: mops.latent_prep(lp, 0, 0, H * d, R, p, dims, None, wkv, c, b.slot_mapping, b.q_start, b.ctx_len, b.seq_of_token,
+                                                      r.inv_freq, r.mscale, 1e-6)
+        sec, lsec = timed(lambda: prep(cache, 0, rot, 0)), timed(lambda: prep(cacheP, P, rotP, P))
+        rec("latent_prep_" + name, sec, "latent_prep with a rotated part of 64", lsec, bytes_=T * R * 4, lbytes=T * (R + P) * 4)
+        # ---- the feed-forward's activation into the joined rows; the joined output product -----------------------------------------------
+        gu, joined = rn(T, 2 * ff), rn(T, H * d + ff)
+        sec = timed(lambda: mops.act_and_mul(gu, mops.ACT_SILU, joined[:, H * d:]))
+        lsec = timed(lambda: mops.act_and_mul(gu, mops.ACT_SILU))
+        rec("act_and_mul_into_rows_" + name, sec, "act_and_mul", lsec, bytes_=T * ff * 6)
+        wj = rn(W, H * d + ff) * ff ** -0.5
+        wo, wd, y2 = wj[:, :H * d].contiguous(), wj[:, H * d:].contiguous(), rn(T, ff)
+        lin = torch.nn.functional.linear
+        sec, lsec = timed(lambda: lin(joined, wj)), timed(lambda: (lin(o, wo), lin(y2, wd)))
+        if name == "prefill":
+            rec("joined_output_product_prefill", sec, "two library products", lsec, flops=2.0 * T * W * (H * d + ff))
+        else:
+            rec("joined_output_product_decode", sec, "two library products", lsec, bytes_=2.0 * W * (H * d + ff))
+    return out
+
+
+def main_vivisun(args) -> int:
+    from . import _lib
+    from .fekotar import FekotarConfig, FekotarForCausalLM
+    from .model import LlamaConfig, LlamaForCausalLM
+    from .vivisun import VivisunConfig, VivisunForCausalLM
+    _lib.lib()
+    _lib.mixers_lib()
+    device = torch.device("cuda", 0)
+    torch.cuda.set_device(device)
+    prompt_len, batch, ctx = args.mixers_prompt, args.batch, args.ctx
+    result = {"metric": "vivisun_vs_llama_bf16_throughput", "unit": "tokens/s", "dtype": "bf16", "data": "synthetic",
+              "n_gpus": 1, "layers": LAYERS, "sizes": {}}
+
+    def llama(s):
+        lc = LlamaConfig(hidden_size=s["width"], intermediate_size=s["ff"], num_hidden_layers=LAYERS,
+                         num_attention_heads=s["heads"], num_key_value_heads=s["kv_heads"], vocab_size=VOCAB,
+                         max_position_embeddings=max(8192, prompt_len + 16))
+        m = LlamaForCausalLM(lc, None, torch.bfloat16).init_synthetic(device)
+        m.use_fused_decode = False
+        return m
+    makers = {"vivisun": lambda s: VivisunForCausalLM(VivisunConfig.from_dict(vivisun_config(s)), torch.bfloat16).init_synthetic(device),
+              "fekotar": lambda s: FekotarForCausalLM(FekotarConfig.from_dict(fekotar_config(s)), torch.bfloat16).init_synthetic(device),
+              "llama": llama}
+    with torch.no_grad():
+        for name, s in SIZES.items():
+            if args.mixers_size and name != args.mixers_size:
+                continue
+            t0 = time.time()
+            r = {who: model_throughput(make(s), prompt_len, batch, ctx, device, VOCAB) for who, make in makers.items()}
+            r["kernels"] = vivisun_kernel_section(s, prompt_len, batch, ctx, device)
+            r["seconds"] = round(time.time() - t0, 1)
+            result["sizes"][name] = r
+            torch.cuda.empty_cache()
+    print(json.dumps(result), flush=True)
+    return 0
+
+
 def main(args) -> int:
     from . import _lib
+    if getattr(args, "mixers_design", "fatudra") == "vivisun":
+        return main_vivisun(args)
     if getattr(args, "mixers_design", "fatudra") == "pagulix":
         return main_pagulix(args)
     if getattr(args, "mixers_design", "fatudra") == "nukezen":

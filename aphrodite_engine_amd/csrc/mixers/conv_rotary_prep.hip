@@ -66,6 +66,38 @@ __device__ __forceinline__ void cr_store8(typename T::storage* p, const float* v
   }
 }
 
+// 8 numbers as they lie in memory (16 bytes of bf16, 32 of fp32): rows in flight take no more registers than that
+template <typename T>
+struct CRChunk {
+  u32x4 v[sizeof(typename T::storage) / 2];
+  __device__ __forceinline__ void load(const typename T::storage* p) {
+#pragma unroll
+    for (int i = 0; i < (int)(sizeof(typename T::storage) / 2); ++i) v[i] = reinterpret_cast<const u32x4*>(p)[i];
+  }
+  __device__ __forceinline__ void clear() {
+#pragma unroll
+    for (int i = 0; i < (int)(sizeof(typename T::storage) / 2); ++i) v[i] = u32x4{0, 0, 0, 0};
+  }
+  __device__ __forceinline__ void store(typename T::storage* p) const {
+#pragma unroll
+    for (int i = 0; i < (int)(sizeof(typename T::storage) / 2); ++i) reinterpret_cast<u32x4*>(p)[i] = v[i];
+  }
+  __device__ __forceinline__ void floats(float* o) const {
+    if constexpr (sizeof(typename T::storage) == 2) {
+      const u16x8 x = __builtin_bit_cast(u16x8, v[0]);
+#pragma unroll
+      for (int j = 0; j < 8; ++j) o[j] = T::to_f32(x[j]);
+    } else {
+      const f32x4 a = __builtin_bit_cast(f32x4, v[0]), b = __builtin_bit_cast(f32x4, v[1]);
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        o[j] = a[j];
+        o[4 + j] = b[j];
+      }
+    }
+  }
+};
+
 constexpr int CR_THREADS = 256, CR_MAX_DIM = 512;
 
 // LDS written by lanes of a wave and read by others of the same wave
@@ -83,6 +115,22 @@ __global__ __launch_bounds__(CR_THREADS) void conv_rotary_qk_norm_kv_write_kerne
   f32x2* turn = reinterpret_cast<f32x2*>(cr_lds + 8 * CR_THREADS);      // (cos, sin) of [row of the tile][pair]
   const int64_t t0 = (int64_t)blockIdx.x * TOK;
   const int half = p.rot_dims >> 1;
+  // what the rows of the tile are (uniform over the workgroup), asked for together
+  int seq[TOK], back0[TOK], ctx[TOK], sslot[TOK];
+  int64_t cslot[TOK];
+#pragma unroll
+  for (int k = 0; k < TOK; ++k) {
+    const int64_t t = t0 + k < p.num_tokens ? t0 + k : p.num_tokens - 1;
+    seq[k] = p.seq_of_token[t];
+    cslot[k] = p.slot_mapping[t];
+  }
+#pragma unroll
+  for (int k = 0; k < TOK; ++k) {
+    const int64_t t = t0 + k < p.num_tokens ? t0 + k : p.num_tokens - 1;
+    back0[k] = (int)t - p.q_start[seq[k]];                   // rows of the segment ahead of this one
+    ctx[k] = p.ctx_len[seq[k]];
+    sslot[k] = TAPS > 1 ? p.state_slots[seq[k]] : 0;
+  }
   for (int i = threadIdx.x; i < TOK * half; i += CR_THREADS) {
     const int64_t t = t0 + i / half;
     if (t >= p.num_tokens) break;
@@ -100,7 +148,8 @@ __global__ __launch_bounds__(CR_THREADS) void conv_rotary_qk_norm_kv_write_kerne
   const int C = (H + G) * p.dim + G * p.vdim;
   const int c0 = (is_v ? (H + G) * p.dim + hd * p.vdim : unit * p.dim) + i0;       // first channel (meaningful if work)
   const bool work = i0 < n;
-  float wv[TAPS][8], nw[8], rows[TOK + TAPS - 1][8];
+  float wv[TAPS][8], nw[8];
+  CRChunk<T> rows[TOK + TAPS - 1];
 #pragma unroll
   for (int i = 0; i < 8; ++i) nw[i] = 1.f;
 #pragma unroll
@@ -120,45 +169,39 @@ __global__ __launch_bounds__(CR_THREADS) void conv_rotary_qk_norm_kv_write_kerne
 #pragma unroll
   for (int x = 0; x < TOK + TAPS - 1; ++x) {
     const int64_t gr = t0 - (TAPS - 1) + x;
-    if (work && gr >= 0 && gr < p.num_tokens) {
-      cr_load8<T>(p.u + gr * p.u_stride + c0, rows[x]);
-    } else {
-#pragma unroll
-      for (int i = 0; i < 8; ++i) rows[x][i] = 0.f;
-    }
+    if (work && gr >= 0 && gr < p.num_tokens) rows[x].load(p.u + gr * p.u_stride + c0);
+    else rows[x].clear();
   }
 #pragma unroll
   for (int k = 0; k < TOK; ++k) {
     const int64_t t = t0 + k;
     if (t >= p.num_tokens) break;
-    const int s = p.seq_of_token[t];
-    const int r = (int)t - p.q_start[s], ctx = p.ctx_len[s];
-    S* st = TAPS > 1 && work ? p.state + (int64_t)p.state_slots[s] * (TAPS - 1) * C + c0 : nullptr;
-    float acc[8], win[TAPS][8];
+    S* st = TAPS > 1 && work ? p.state + (int64_t)sslot[k] * (TAPS - 1) * C + c0 : nullptr;
+    float acc[8];
+    CRChunk<T> win[TAPS];
 #pragma unroll
     for (int j = 0; j < TAPS; ++j) {
-      const int back = r - TAPS + 1 + j;                     // row of the segment, negative: before it
-      if (back >= 0) {
-#pragma unroll
-        for (int i = 0; i < 8; ++i) win[j][i] = rows[k + j][i];
-      } else if (work && ctx + back >= 0) {
-        cr_load8<T>(st + (int64_t)(TAPS - 1 + back) * C, win[j]);
-      } else {
-#pragma unroll
-        for (int i = 0; i < 8; ++i) win[j][i] = 0.f;
+      const int back = back0[k] - TAPS + 1 + j;              // row of the segment, negative: before it
+      win[j] = rows[k + j];
+      if (back < 0) {
+        if (work && ctx[k] + back >= 0) win[j].load(st + (int64_t)(TAPS - 1 + back) * C);
+        else win[j].clear();
       }
     }
 #pragma unroll
-    for (int i = 0; i < 8; ++i) {
-      acc[i] = 0.f;
+    for (int i = 0; i < 8; ++i) acc[i] = 0.f;
 #pragma unroll
-      for (int j = 0; j < TAPS; ++j) acc[i] += wv[j][i] * win[j][i];
+    for (int j = 0; j < TAPS; ++j) {
+      float x[8];
+      win[j].floats(x);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) acc[i] += wv[j][i] * x[i];
     }
     if (p.write_state && work) {
 #pragma unroll
-      for (int m = 0; m < TAPS - 1; ++m) cr_store8<T>(st + (int64_t)m * C, win[m + 1]);
+      for (int m = 0; m < TAPS - 1; ++m) win[m + 1].store(st + (int64_t)m * C);
     }
-    const int64_t slot = p.slot_mapping[t];
+    const int64_t slot = cslot[k];
     const bool cached = slot >= 0 && slot < p.num_cache_rows;
     if (is_v) {
       if (work && cached) cr_store8<T>(p.v_cache + (slot * G + hd) * (int64_t)p.vdim + i0, acc);

@@ -36,10 +36,12 @@ bool dba_decode_supported(int heads, int kv_heads, int dim, int vdim);
 // workgroups per decoded row (before the key range is split)
 int dba_decode_units(int heads, int kv_heads, int dim, int vdim);
 int dba_decode_splits(int64_t num_tokens, int units, int max_kv_len, int64_t ws_floats, int heads, int vdim);
-// EXT: window / chunk, soft cap, sink, elementwise gate (a translation unit each)
-template <bool EXT>
+// The forms of the kernels, a translation unit each: causal with a gate per head at most; window / chunk, soft cap, sink and elementwise
+// gate, chosen at run time; causal with an elementwise gate.
+enum DBAForm { DBA_PLAIN = 0, DBA_MASKED = 1, DBA_GATED = 2 };
+template <int FORM>
 void dba_prefill_launch(const DBAParams& p, int max_q_len, int num_seqs, hipStream_t st);
-template <bool EXT>
+template <int FORM>
 void dba_decode_launch(const DBAParams& p, int64_t num_tokens, int nsplit, hipStream_t st);
 constexpr int DBA_MFMA_MIN_LEN = 8;     // segments at least this long go to the matrix-core kernel
 

@@ -205,7 +205,7 @@ extern "C" int aphro_distance_bias_attention(void* out, int64_t out_stride, cons
   APHRO_CHECK(temp_coef == 0.f || temp_every > 0, "distance_bias_attention: temp_every must be positive");
   APHRO_CHECK(window >= 0 && chunk >= 0 && softcap >= 0.f && (gate_cols == 0 || gate_cols == 1), "distance_bias_attention: window %d, chunk %d, cap %g",
               window, chunk, softcap);
-  const bool ext = window > 0 || chunk > 0 || softcap > 0.f || sink || (gate && gate_cols);
+  const int form = window > 0 || chunk > 0 || softcap > 0.f || sink ? DBA_MASKED : (gate && gate_cols ? DBA_GATED : DBA_PLAIN);
   int visible = max_kv_len;                                 // what a row can see, not how long its sequence is, decides the split
   if (window > 0) visible = min(visible, window);
   if (chunk > 0) visible = min(visible, chunk);
@@ -233,19 +233,22 @@ extern "C" int aphro_distance_bias_attention(void* out, int64_t out_stride, cons
     const bool all_long = min_q_len >= DBA_MFMA_MIN_LEN;
     if (pf && (all_long || dc)) {
       p.min_len = DBA_MFMA_MIN_LEN;
-      if (ext) dba_prefill_launch<true>(p, max_q_len, num_seqs, (hipStream_t)stream);
-      else dba_prefill_launch<false>(p, max_q_len, num_seqs, (hipStream_t)stream);
+      if (form == DBA_MASKED) dba_prefill_launch<DBA_MASKED>(p, max_q_len, num_seqs, (hipStream_t)stream);
+      else if (form == DBA_GATED) dba_prefill_launch<DBA_GATED>(p, max_q_len, num_seqs, (hipStream_t)stream);
+      else dba_prefill_launch<DBA_PLAIN>(p, max_q_len, num_seqs, (hipStream_t)stream);
       if (!all_long) {
-        if (ext) dba_decode_launch<true>(p, num_tokens, nsplit, (hipStream_t)stream);
-        else dba_decode_launch<false>(p, num_tokens, nsplit, (hipStream_t)stream);
+        if (form == DBA_MASKED) dba_decode_launch<DBA_MASKED>(p, num_tokens, nsplit, (hipStream_t)stream);
+        else if (form == DBA_GATED) dba_decode_launch<DBA_GATED>(p, num_tokens, nsplit, (hipStream_t)stream);
+        else dba_decode_launch<DBA_PLAIN>(p, num_tokens, nsplit, (hipStream_t)stream);
       }
       APHRO_LAUNCH_CHECK();
       return APHRO_OK;
     }
     if (dc) {
       p.min_len = 0x7fffffff;
-      if (ext) dba_decode_launch<true>(p, num_tokens, nsplit, (hipStream_t)stream);
-      else dba_decode_launch<false>(p, num_tokens, nsplit, (hipStream_t)stream);
+      if (form == DBA_MASKED) dba_decode_launch<DBA_MASKED>(p, num_tokens, nsplit, (hipStream_t)stream);
+      else if (form == DBA_GATED) dba_decode_launch<DBA_GATED>(p, num_tokens, nsplit, (hipStream_t)stream);
+      else dba_decode_launch<DBA_PLAIN>(p, num_tokens, nsplit, (hipStream_t)stream);
       APHRO_LAUNCH_CHECK();
       return APHRO_OK;
     }

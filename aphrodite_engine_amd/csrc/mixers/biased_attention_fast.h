@@ -1,7 +1,8 @@
 // bf16 fast paths of the distance-biased attention (same semantics as biased_attention.hip, which stays the fp32 path and
-// the path of sizes these do not tile).  EXT adds, at run time: a sliding window or chunks (both give every row an oldest key;
+// the path of sizes these do not tile).  EXT (the form DBA_MASKED) adds, at run time: a sliding window or chunks (both give every row an oldest key;
 // key tiles older than that are not visited), a tanh soft cap on the scores, a per-head sink in the denominator and an
-// elementwise gate.  The plain forms and the EXT forms are translation units of their own.
+// elementwise gate.  DBA_GATED is the plain form with the elementwise gate (and none of
+// the branches of the masked loop).  Every form is a translation unit of its own.
 //
 //  * dba_prefill_kernel<DK, DV>: segments of >= DBA_MFMA_MIN_LEN rows.  A workgroup of four waves owns 64 consecutive
 //    query rows of one (segment, head), 16 rows per wave, and walks the visible keys 64 at a time: the K rows and V rows of
@@ -56,11 +57,12 @@ __device__ __forceinline__ float dba_cap2(const DBAParams& p, float x) {
 }
 
 // a decoded row's column: o = sum of e^(s - M) v, L = sum of e^(s - M); sink, gate, scale and store
-template <bool EXT>
+template <int FORM>
 __device__ __forceinline__ void dba_finish(const DBAParams& p, int t, int head, int col, float M, float L, float o) {
+  constexpr bool EXT = FORM == DBA_MASKED;
   float sig = p.out_scale;
   if (p.gate) {
-    const int at = EXT && p.gate_cols ? head * p.vdim + col : head;
+    const int at = FORM != DBA_PLAIN && p.gate_cols ? head * p.vdim + col : head;
     sig *= sigmoid_f(BFloat::to_f32(p.gate[(int64_t)t * p.gate_stride + at]));
   }
   if (EXT && p.sink) {
@@ -138,8 +140,9 @@ __device__ __forceinline__ void pf_store(const PFStage<DK, DV>& st, uint16_t* k_
 
 // QT query heads of one kv head share a workgroup: the K and V fragments read from LDS feed QT products each, and the
 // tile's trip from the cache to LDS is paid once for them.
-template <int DK, int DV, int QT, bool EXT>
+template <int DK, int DV, int QT, int FORM>
 __global__ __launch_bounds__(256) void dba_prefill_kernel(DBAParams p) {
+  constexpr bool EXT = FORM == DBA_MASKED;
   constexpr int NCHK = DK / 8, NKS = DK / 32, NDT = DV / 16, NH = PF_BN / 16, NPK = PF_BN / 32;
   constexpr int SWZ = (NCHK & -NCHK) - 1;
   constexpr int NWIN = PF_BM + PF_BN - 1;
@@ -310,9 +313,9 @@ __global__ __launch_bounds__(256) void dba_prefill_kernel(DBAParams p) {
       const float s2 = p.sink[head0 + t] * LOG2E, M = fmaxf(m_run[t], s2), a = __builtin_amdgcn_exp2f(m_run[t] - M);
       f = a / (l * a + __builtin_amdgcn_exp2f(s2 - M)) * p.out_scale;
     }
-    if (p.gate && !(EXT && p.gate_cols)) f *= sigmoid_f(BFloat::to_f32(p.gate[(int64_t)(s0 + qrow) * p.gate_stride + head0 + t]));
+    if (p.gate && !(FORM != DBA_PLAIN && p.gate_cols)) f *= sigmoid_f(BFloat::to_f32(p.gate[(int64_t)(s0 + qrow) * p.gate_stride + head0 + t]));
     uint16_t* op = p.out + (int64_t)(s0 + qrow) * p.out_stride + (head0 + t) * DV;
-    if constexpr (EXT) {
+    if constexpr (FORM != DBA_PLAIN) {
       const uint16_t* gp = p.gate && p.gate_cols ? p.gate + (int64_t)(s0 + qrow) * p.gate_stride + (head0 + t) * DV : nullptr;
 #pragma unroll
       for (int dt = 0; dt < NDT; ++dt) {
@@ -342,8 +345,9 @@ __global__ __launch_bounds__(256) void dba_prefill_kernel(DBAParams p) {
   }
 }
 
-template <int QH, int CHL, bool EXT>
+template <int QH, int CHL, int FORM>
 __global__ __launch_bounds__(256) void dba_decode_kernel(DBAParams p) {
+  constexpr bool EXT = FORM == DBA_MASKED;
   constexpr int CH = 1 << CHL;       // lanes per key row (16 bytes each)
   constexpr int KP = 64 / CH;        // keys per load instruction
   constexpr int NI = 4;              // load instructions per step of the online softmax (few: registers buy occupancy)
@@ -486,11 +490,11 @@ __global__ __launch_bounds__(256) void dba_decode_kernel(DBAParams p) {
       w[2 + col] = o;
       continue;
     }
-    dba_finish<EXT>(p, t, head, col, M, L, o);
+    dba_finish<FORM>(p, t, head, col, M, L, o);
   }
 }
 
-template <bool EXT>
+template <int FORM>
 __global__ void dba_merge_kernel(DBAParams p, int nsplit) {
   const int t = blockIdx.x, head = blockIdx.y;
   if (p.q_len[p.seq_of_token[t]] >= p.min_len) return;
@@ -508,39 +512,39 @@ __global__ void dba_merge_kernel(DBAParams p, int nsplit) {
       const float mz = w[z * (2 + p.vdim)];
       if (mz != -INFINITY) o += w[z * (2 + p.vdim) + 2 + col] * __expf(mz - M);
     }
-    dba_finish<EXT>(p, t, head, col, M, L, o);
+    dba_finish<FORM>(p, t, head, col, M, L, o);
   }
 }
 
-template <int DK, int QT, bool EXT>
+template <int DK, int QT, int FORM>
 static void launch_prefill_dv(const DBAParams& p, dim3 grid, hipStream_t st) {
   switch (p.vdim) {
-    case 32: hipLaunchKernelGGL((dba_prefill_kernel<DK, 32, QT, EXT>), grid, dim3(256), 0, st, p); break;
-    case 64: hipLaunchKernelGGL((dba_prefill_kernel<DK, 64, QT, EXT>), grid, dim3(256), 0, st, p); break;
-    case 96: hipLaunchKernelGGL((dba_prefill_kernel<DK, 96, QT, EXT>), grid, dim3(256), 0, st, p); break;
-    case 128: hipLaunchKernelGGL((dba_prefill_kernel<DK, 128, QT, EXT>), grid, dim3(256), 0, st, p); break;
+    case 32: hipLaunchKernelGGL((dba_prefill_kernel<DK, 32, QT, FORM>), grid, dim3(256), 0, st, p); break;
+    case 64: hipLaunchKernelGGL((dba_prefill_kernel<DK, 64, QT, FORM>), grid, dim3(256), 0, st, p); break;
+    case 96: hipLaunchKernelGGL((dba_prefill_kernel<DK, 96, QT, FORM>), grid, dim3(256), 0, st, p); break;
+    case 128: hipLaunchKernelGGL((dba_prefill_kernel<DK, 128, QT, FORM>), grid, dim3(256), 0, st, p); break;
   }
 }
 
-template <int QT, bool EXT>
+template <int QT, int FORM>
 static void launch_prefill_dk(const DBAParams& p, dim3 grid, hipStream_t st) {
   switch (p.dim) {
-    case 32: launch_prefill_dv<32, QT, EXT>(p, grid, st); break;
-    case 64: launch_prefill_dv<64, QT, EXT>(p, grid, st); break;
-    case 96: launch_prefill_dv<96, QT, EXT>(p, grid, st); break;
-    case 128: launch_prefill_dv<128, QT, EXT>(p, grid, st); break;
+    case 32: launch_prefill_dv<32, QT, FORM>(p, grid, st); break;
+    case 64: launch_prefill_dv<64, QT, FORM>(p, grid, st); break;
+    case 96: launch_prefill_dv<96, QT, FORM>(p, grid, st); break;
+    case 128: launch_prefill_dv<128, QT, FORM>(p, grid, st); break;
   }
 }
 
-template <bool EXT>
+template <int FORM>
 void dba_prefill_launch(const DBAParams& p0, int max_q_len, int num_seqs, hipStream_t st) {
   DBAParams p = p0;
   p.max_tiles = (max_q_len + PF_BM - 1) / PF_BM;
   const int qt = (p.heads / p.kv_heads) % 2 == 0 ? 2 : 1;   // two query heads of a kv head per workgroup where they pair up
   const int per_seq = (p.max_tiles * (p.heads / qt) + 7) / 8 * 8;      // a multiple of the XCD count: the numbering repeats per segment
   const dim3 grid((unsigned)per_seq, (unsigned)num_seqs);
-  if (qt == 2) launch_prefill_dk<2, EXT>(p, grid, st);
-  else launch_prefill_dk<1, EXT>(p, grid, st);
+  if (qt == 2) launch_prefill_dk<2, FORM>(p, grid, st);
+  else launch_prefill_dk<1, FORM>(p, grid, st);
 }
 
 // lanes per key row: the smallest power of two that covers both row lengths in 16-byte pieces
@@ -559,11 +563,11 @@ static int decode_qh(int heads, int kv_heads, int chl) {
   return qh;
 }
 
-template <bool EXT>
+template <int FORM>
 void dba_decode_launch(const DBAParams& p, int64_t num_tokens, int nsplit, hipStream_t st) {
   const dim3 grid((unsigned)num_tokens, (unsigned)dba_decode_units(p.heads, p.kv_heads, p.dim, p.vdim), (unsigned)nsplit);
   const int chl = decode_chl(p.dim, p.vdim), qh = decode_qh(p.heads, p.kv_heads, chl);
-#define DEC(QH, CHL) hipLaunchKernelGGL((dba_decode_kernel<QH, CHL, EXT>), grid, dim3(256), 0, st, p)
+#define DEC(QH, CHL) hipLaunchKernelGGL((dba_decode_kernel<QH, CHL, FORM>), grid, dim3(256), 0, st, p)
 #define DEC_BY_CHL(QH)                          \
   switch (chl) {                                \
     case 2: DEC(QH, 2); break;                  \
@@ -580,7 +584,7 @@ void dba_decode_launch(const DBAParams& p, int64_t num_tokens, int nsplit, hipSt
 #undef DEC_BY_CHL
 #undef DEC
   if (nsplit > 1)
-    hipLaunchKernelGGL((dba_merge_kernel<EXT>), dim3((unsigned)num_tokens, (unsigned)p.heads), dim3(64), 0, st, p, nsplit);
+    hipLaunchKernelGGL((dba_merge_kernel<FORM>), dim3((unsigned)num_tokens, (unsigned)p.heads), dim3(64), 0, st, p, nsplit);
 }
 
 }  // namespace aphro

@@ -27,7 +27,7 @@ int dba_decode_splits(int64_t num_tokens, int units, int max_kv_len, int64_t ws_
   return n < 1 ? 1 : (int)n;
 }
 
-template void dba_prefill_launch<false>(const DBAParams&, int, int, hipStream_t);
-template void dba_decode_launch<false>(const DBAParams&, int64_t, int, hipStream_t);
+template void dba_prefill_launch<DBA_PLAIN>(const DBAParams&, int, int, hipStream_t);
+template void dba_decode_launch<DBA_PLAIN>(const DBAParams&, int64_t, int, hipStream_t);
 
 }  // namespace aphro

@@ -3,7 +3,7 @@
 
 namespace aphro {
 
-template void dba_prefill_launch<true>(const DBAParams&, int, int, hipStream_t);
-template void dba_decode_launch<true>(const DBAParams&, int64_t, int, hipStream_t);
+template void dba_prefill_launch<DBA_MASKED>(const DBAParams&, int, int, hipStream_t);
+template void dba_decode_launch<DBA_MASKED>(const DBAParams&, int64_t, int, hipStream_t);
 
 }  // namespace aphro
